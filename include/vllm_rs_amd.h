@@ -703,7 +703,7 @@ void vra_stack_op_sandwich_norm(float* x, const float* p1, int32_t n1, const flo
 
 /* attention_window: the softmax attention under a sliding window (key j visible iff 0 <= p_i - j < window; 0 = causal), with a sink per head
  * in the denominator, a scale per head on the scores and sigmoid(gate[t, h]) on head h's output row (null pointers: absent).
- * seam: vra_stack_op_sandwich_norm with Dynamic Tanh norms (dyt = 1: tanh(alpha v) w + b), an RMS norm of its own per part (p1_norm_w /
+ * seam: vra_stack_op_sandwich_norm with a choice of norm (norm_kind 0 RMS, 1 Dynamic Tanh tanh(alpha v) w + b, 2 layer norm), an RMS norm of its own per part (p1_norm_w /
  * p2_norm_w), pairs without a row (pe < 0), a per-row weight on the second part (p2w), the unrounded h (h32), and router_kind 1: softmax
  * over all n_router outputs, router_bias added for the choice only, choice within the `keep` best of n_groups groups, weights = scores,
  * the last n_identity outputs chosen as expert -1 with their weights summed into id_weight.
@@ -717,7 +717,7 @@ void vra_stack_op_attention_window(const void* q, int32_t ldq, void* out, const 
                                    float scale, int32_t window, const float* sink, const float* head_scale, const float* gate,
                                    int32_t gate_ld, int32_t dtype, int64_t stream);
 void vra_stack_op_seam(float* x, const float* p1, int32_t n1, const float* pw, const int32_t* pe, float c1, const float* p2, const float* p2w,
-                       float c2, const float* p1_norm_w, const float* p2_norm_w, int32_t dyt, const float* post_w, const float* post_b,
+                       float c2, const float* p1_norm_w, const float* p2_norm_w, int32_t norm_kind, const float* post_w, const float* post_b,
                        float post_alpha, const float* pre_w, const float* pre_b, float pre_alpha, void* h, float* h32, float eps, int32_t T,
                        int32_t W, const void* router_w, const float* router_bias, int32_t router_kind, int32_t n_router, int32_t top,
                        int32_t n_groups, int32_t keep, int32_t n_identity, int32_t* pair_expert, float* pair_weight, float* id_weight,

@@ -93,7 +93,7 @@ def test_native_parser_accepts_the_layer_list():
     (lambda s: s.replace("heads=4 ", "heads=3 ", 1), "multiple of kv_heads"),
     (lambda s: s.replace("rot_dims=4", "rot_dims=6", 1), "rot_dims"),
     (lambda s: s.replace("block=sequential", "block=parallel"), "sequential blocks"),
-    (lambda s: s.replace("norm=dyt", "norm=layer"), "norm must be"),
+    (lambda s: s.replace("norm=dyt", "norm=batch"), "norm must be"),
     (lambda s: s.replace("mixer=latent", "mixer=conv", 1), "unknown mixer"),
 ])
 def test_native_parser_refuses_inconsistent_lists(edit, why):

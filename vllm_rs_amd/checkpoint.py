@@ -266,7 +266,54 @@ def parse_sudosun(cfg_json, dtype=None):
                 rms_norm_eps=float(norm.get("eps", 1e-6)), rope_theta=10000.0, dtype=dt, quant_method=None, spec="\n".join(lines) + "\n")
 
 
-STACK_ARCHS = {"Ditilix": parse_ditilix, "Gaperax": parse_gaperax, "Zifetar": parse_zifetar, "Sudosun": parse_sudosun}
+def parse_pesivik(cfg_json, dtype=None):
+    """Pesivik config.json -> cfg dict with arch "stack": sandwich blocks with layer norms and a scale per channel on each sub-block's normed
+    output, a scaled embedding, latent attention under a sliding window (rotate-half rotary part, one output gate per head), a mixture of
+    experts without gates (sigmoid router, corrected choice among the best groups, normalised weights, a shared expert) or no feed-forward,
+    capped logits, optionally the tensors of another layer ("weights_of").  Every size and constant comes from the config."""
+    td = dtype or cfg_json.get("torch_dtype", "bfloat16")
+    dt = {"bfloat16": BF16, "bf16": BF16, "float32": F32, "f32": F32, BF16: BF16, F32: F32}.get(td)
+    if dt is None:
+        raise ValueError(f"dtype {td!r}: a layer stack runs in bfloat16 or float32")
+    norm = cfg_json.get("norm") or {}
+    width, vocab, layers = int(cfg_json["width"]), int(cfg_json["vocab"]), cfg_json["layers"]
+    lines = ["stack width=%d vocab=%d eps=%s block=sandwich norm=layer pos=none layer_scale=1 embed_scale=%s logit_softcap=%s" % (
+        width, vocab, _num(norm.get("eps", 1e-5)), _num((cfg_json.get("embedding") or {}).get("scale", 1.0)), _num(cfg_json.get("logit_softcap") or 0.0))]
+    heads = dim = 1
+    for i, layer in enumerate(layers):
+        if layer.get("type", "latent_attention") != "latent_attention":
+            raise ValueError(f"layer {i}: mixer type {layer.get('type')!r} is not part of this design")
+        mx = layer["mixer"]
+        rot, rot_dim = mx.get("rot") or {}, int(mx.get("rot_dim", 0))
+        if rot and int(rot.get("dims", rot_dim)) != rot_dim:
+            raise ValueError(f"layer {i}: the rotated part has {rot_dim} dimensions, rot.dims says {rot['dims']}")
+        f = dict(mixer="latent", kv_heads=1, heads=int(mx["heads"]), dim=int(mx["dim"]), vdim=int(mx.get("vdim", mx["dim"])), kv_rank=int(mx["kv_rank"]),
+                 q_rank=int(mx["q_rank"]), rot_dim=rot_dim, rot_dims=rot_dim, rot_base=_num(rot.get("base", 10000.0)), rot_layout="half",
+                 scale=_num(mx["scale"]) if mx.get("scale") is not None else _num((int(mx["dim"]) + rot_dim) ** -0.5),
+                 window=int((mx.get("mask") or {}).get("size", 0)), head_gate=1)
+        if layer.get("weights_of") is not None:
+            f.update(weights_of=int(layer["weights_of"]))
+        mlp = layer.get("mlp")
+        if not mlp:
+            f.update(mlp="none")
+        elif mlp["kind"] == "moe":
+            r = mlp["router"]
+            f.update(mlp="moe", ff=int(mlp["expert"]["ff"]), experts=int(r["experts"]), top=int(r.get("top", 1)), router="sigmoid_norm", act="gelu")
+            g = r.get("groups")
+            if g:
+                f.update(groups=int(g["count"]), keep=int(g["keep"]))
+            if mlp.get("shared"):
+                f.update(shared_ff=int(mlp["shared"]["ff"]))
+        else:
+            raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not part of this design")
+        lines.append("layer " + " ".join(f"{k}={v}" for k, v in f.items()))
+        heads, dim = max(heads, f["heads"]), max(dim, f["dim"], f["vdim"])
+    return dict(arch="stack", design="Pesivik", hidden_size=width, vocab_size=vocab, num_layers=len(layers), num_heads=heads, num_kv_heads=1,
+                head_dim=dim, intermediate_size=0, max_position_embeddings=int(cfg_json.get("max_position_embeddings", 1 << 20)),
+                rms_norm_eps=float(norm.get("eps", 1e-5)), rope_theta=10000.0, dtype=dt, quant_method=None, spec="\n".join(lines) + "\n")
+
+
+STACK_ARCHS = {"Ditilix": parse_ditilix, "Gaperax": parse_gaperax, "Zifetar": parse_zifetar, "Sudosun": parse_sudosun, "Pesivik": parse_pesivik}
 
 
 def parse_config(cfg_json, dtype=None):

@@ -13,6 +13,8 @@
 // epi 0: plain.  epi 1: gated pair — W holds gate and up rows interleaved in blocks of 16 (block 2b = gate rows 16b.., block 2b+1 =
 // up rows 16b..), N counts both; out gets N/2 columns of  g' * sigmoid(act_alpha * g') * (u' + 1),  g' = min(g, limit),
 // u' = clamp(u, -limit, limit)  (limit <= 0: no clamp).
+// epi 2: element-wise activation of a plain product: out = act(alpha * sum + bias), act 3: the exact gelu 0.5 z (1 + erf(z / sqrt 2)).
+// softcap > 0 (plain products): out = softcap * tanh(v / softcap) of the finished value v.
 struct StkGemmArgs {
   const void* a = nullptr;
   int lda = 0;
@@ -30,7 +32,8 @@ struct StkGemmArgs {
   const int* out_row = nullptr;
   int epi = 0;
   float limit = 0.f, act_alpha = 1.702f;
-  int act = 0;                  // the gated pair of epi 1: 0 the clamped form above, 1  gelu_tanh(g) * u, 2  silu(g) * u
+  int act = 0;                  // the gated pair of epi 1: 0 the clamped form above, 1  gelu_tanh(g) * u, 2  silu(g) * u;  epi 2: 3 exact gelu
+  float softcap = 0.f;
   const float* bias = nullptr;  // f32 [N], added after alpha (plain epilogue)
   // batched form (no row groups): product z of `batch` reads a + z * a_batch_stride, w + z * w_batch_stride and writes out + z * out_batch_stride
   // (element counts; a column offset per head turns one launch into a product per head)
@@ -130,6 +133,7 @@ struct StkRotary {
   const float* freq_lo = nullptr;
   int pairs = 0;      // rotated dimensions / 2; the dimensions behind them pass unchanged
   float mag = 1.f;    // multiplies cos and sin
+  int half = 0;       // 1: dimension i pairs with i + pairs (rotate-half layout) instead of 2i with 2i + 1  (latent prep, rope heads)
 };
 
 // Latent projections of one token, from the f32 row  raw = [a | b | r]  of the joint down-projection:
@@ -225,13 +229,15 @@ void vra_stack_embed_pair(const StkEmbedPairArgs& a, int dtype, int64_t stream);
 //   with p1_norm_w / p2_norm_w (n1 = 1): each part is first divided by its root mean square over the row and multiplied by that weight
 //   x[t] += N(s; post_w)                                                              (post_w null: nothing is added)
 //   h[t]  = N(x[t]; pre_w)  in dtype                                                  (pre_w null: no h);  h32: also the unrounded h (f32)
-// N is an RMS norm with a weight, or (dyt) Dynamic Tanh  tanh(alpha v) w + b  with the slopes post_alpha / pre_alpha and offsets post_b / pre_b.
+// N by norm_kind: 0 RMS norm with a weight; 1 Dynamic Tanh  tanh(alpha v) w + b  with the slopes post_alpha / pre_alpha and offsets post_b /
+// pre_b; 2 layer norm  (v - mean) / sqrt(mean((v - mean)^2) + eps) * w  (no offset).
 // With router_w ([n_router, W] in dtype): z = router_w . h + router_bias on the unrounded h, the `top` largest (ties: the lower
 // index) -> pair_expert / pair_weight [T, top].  router_kind 0: weights = softmax over the chosen logits.  router_kind 1: scores =
 // softmax over all n_router logits; the choice goes by score + router_bias (a correction that the weights do not carry) among the experts of
 // the `keep` groups (of n_groups equal groups of neighbours) whose largest corrected score is largest; weights = the chosen scores as they
 // are; the last n_identity router outputs are experts without tensors that hand their input back: their pairs get expert -1 and their
-// weights are summed into id_weight[t].  All f32.
+// weights are summed into id_weight[t].  router_kind 2: as 1, but scores = sigmoid of each logit, a group's worth is the SUM of its two largest
+// corrected scores (a group of one: that score), and the weights are the chosen scores divided by (their sum + 1e-20).  All f32.
 struct StkSandwichArgs {
   float* x = nullptr;
   const float* p1 = nullptr;
@@ -250,7 +256,7 @@ struct StkSandwichArgs {
   int n_router = 0, top = 0;
   int* pair_expert = nullptr;
   float* pair_weight = nullptr;
-  int dyt = 0;
+  int norm_kind = 0;
   const float* post_b = nullptr;
   const float* pre_b = nullptr;
   float post_alpha = 1.f, pre_alpha = 1.f;

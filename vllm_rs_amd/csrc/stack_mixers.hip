@@ -51,10 +51,11 @@ __global__ __launch_bounds__(256) void stk_latent_prep_kernel(StkLatentPrepArgs 
     if (i < a.rot.pairs) {
       float c, sn;
       rot_cos_sin(a.rot, i, p, &c, &sn);
-      const float u = r[2 * i], v = r[2 * i + 1];
-      El<T>::st(row + a.kv_rank + 2 * i, u * c - v * sn);
-      El<T>::st(row + a.kv_rank + 2 * i + 1, v * c + u * sn);
-    } else {
+      const int iu = a.rot.half ? i : 2 * i, iv = a.rot.half ? i + a.rot.pairs : 2 * i + 1;
+      const float u = r[iu], v = r[iv];
+      El<T>::st(row + a.kv_rank + iu, u * c - v * sn);
+      El<T>::st(row + a.kv_rank + iv, v * c + u * sn);
+    } else {  // (behind the rotated dimensions both layouts count on in pairs)
       El<T>::st(row + a.kv_rank + 2 * i, r[2 * i]);
       if (2 * i + 1 < a.rot_dim) El<T>::st(row + a.kv_rank + 2 * i + 1, r[2 * i + 1]);
     }
@@ -74,9 +75,10 @@ __global__ __launch_bounds__(256) void stk_rope_heads_kernel(const T* in, int in
     if (i < rot.pairs) {
       float c, sn;
       rot_cos_sin(rot, i, p, &c, &sn);
-      const float u = El<T>::ld(src + 2 * i), v = El<T>::ld(src + 2 * i + 1);
-      El<T>::st(dst + 2 * i, u * c - v * sn);
-      El<T>::st(dst + 2 * i + 1, v * c + u * sn);
+      const int iu = rot.half ? i : 2 * i, iv = rot.half ? i + rot.pairs : 2 * i + 1;
+      const float u = El<T>::ld(src + iu), v = El<T>::ld(src + iv);
+      El<T>::st(dst + iu, u * c - v * sn);
+      El<T>::st(dst + iv, v * c + u * sn);
     } else {
       El<T>::st(dst + 2 * i, El<T>::ld(src + 2 * i));
       if (2 * i + 1 < n) El<T>::st(dst + 2 * i + 1, El<T>::ld(src + 2 * i + 1));

@@ -13,6 +13,13 @@
 namespace {
 
 __device__ __forceinline__ float gelu_tanh_(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
+__device__ __forceinline__ float gelu_erf_(float z) { return 0.5f * z * (1.f + erff(z * 0.7071067811865476f)); }
+// the finished value of a plain product: element-wise activation (epi 2), soft cap
+__device__ __forceinline__ float plain_value(const StkGemmArgs& g, float v) {
+  if (g.epi == 2) v = gelu_erf_(v);
+  if (g.softcap > 0.f) v = g.softcap * tanhf(v / g.softcap);
+  return v;
+}
 // act 0: min(g, L) * sigmoid(act_alpha * min(g, L)) * (clamp(u, +-L) + 1);  act 1: gelu_tanh(g) * u;  act 2: silu(g) * u
 __device__ __forceinline__ float gated_pair(float g, float u, float limit, float act_alpha, int act = 0) {
   if (act == 1) return gelu_tanh_(g) * u;
@@ -206,7 +213,7 @@ __global__ __launch_bounds__(256) void stk_gemm_simple_kernel(StkGemmArgs g) {
     for (int j = 0; j < 4; j++) {
       const int n = n0 + tx * 4 + j;
       if (n >= g.N) continue;
-      const float v = acc[i][j] * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f);
+      const float v = plain_value(g, acc[i][j] * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f));
       if (g.out_f32) ((float*)g.out)[ob + (int64_t)orow * g.ldo + n] = v;
       else El<T>::st((T*)g.out + ob + (int64_t)orow * g.ldo + n, v);
     }
@@ -217,7 +224,8 @@ __global__ __launch_bounds__(256) void stk_gemm_simple_kernel(StkGemmArgs g) {
 // A wave owns MT x NT tiles of 16 x 16; both operands come straight from global memory in the instruction's operand order (lane =
 // (row rq = lane & 15, k octet oct = lane >> 4): 16 bytes of one row per lane and K-step of 32), the weights as the A operand and the
 // activations as B, so a lane ends up with 4 consecutive output columns of ONE activation row.  K ascending in steps of 32.
-template <int MT, int NT, int WM, int WN, bool SCALED>
+// POST: the plain epilogue also applies an activation or a soft cap
+template <int MT, int NT, int WM, int WN, bool SCALED, bool POST = false>
 __global__ __launch_bounds__(64 * WM * WN) void stk_gemm_mfma_kernel(StkGemmArgs g) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int wm = wave % WM, wn = wave / WM, rq = lane & 15, oct = lane >> 4;
@@ -315,7 +323,8 @@ __global__ __launch_bounds__(64 * WM * WN) void stk_gemm_mfma_kernel(StkGemmArgs
         for (int j = 0; j < 4; j++) {
           const int n = n_base + nt * 16 + oct * 4 + j;
           if (n >= g.N) continue;
-          const float v = acc[mt][nt][j] * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f);
+          float v = acc[mt][nt][j] * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f);
+          if (POST) v = plain_value(g, v);
           if (g.out_f32) ((float*)g.out)[ob + (int64_t)orow * g.ldo + n] = v;
           else ((uint16_t*)g.out)[ob + (int64_t)orow * g.ldo + n] = BF16::from_f32(v);
         }
@@ -326,7 +335,7 @@ __global__ __launch_bounds__(64 * WM * WN) void stk_gemm_mfma_kernel(StkGemmArgs
 // Steps of up to 32 rows (decoding): the weights are the whole traffic, so a workgroup takes only 32 output columns and its 8 waves
 // take an eighth of K each (whole K-steps of 32, ascending inside a wave); the 8 partial tiles meet in LDS and are summed in wave order.
 // One fixed order for a given K — another one than the large-M kernel's single chain, so the two agree to rounding, not to the bit.
-template <bool SCALED>
+template <bool SCALED, bool POST = false>
 __global__ __launch_bounds__(512) void stk_gemm_mfma_small_kernel(StkGemmArgs g) {
   __shared__ float part[8][16 * 32];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, rq = lane & 15, oct = lane >> 4;
@@ -401,7 +410,8 @@ __global__ __launch_bounds__(512) void stk_gemm_mfma_small_kernel(StkGemmArgs g)
   } else {
     const int n = n_base + c;
     if (n >= g.N) return;
-    const float v = total(c) * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f);
+    float v = total(c) * g.alpha + (g.bias ? g.bias[(int64_t)blockIdx.z * g.bias_batch_stride + n] : 0.f);
+    if (POST) v = plain_value(g, v);
     if (g.out_f32) ((float*)g.out)[ob + (int64_t)orow * g.ldo + n] = v;
     else ((uint16_t*)g.out)[ob + (int64_t)orow * g.ldo + n] = BF16::from_f32(v);
   }
@@ -511,7 +521,7 @@ __device__ __forceinline__ float cap_score_fast(float s, float softcap) {
 // tokens staged once in LDS (f32) for all 16 rows; lane = key for the scores, lane = value channel for the weighted sum.
 // Tiles start at key 0 of the sequence and a row's running maximum / sum go tile by tile: the order does not depend on the portion.
 #define STK_QT 16
-template <typename T, int KT>
+template <typename T, int KT, int NR>
 __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   extern __shared__ float lds[];
   const int dim = a.dim, vdim = a.vdim, kld = dim + 1;
@@ -546,11 +556,11 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   for (int r = 0; r < nq; r++) pmax = max(pmax, a.positions[t0 + r]), lo_min = min(lo_min, block_start(a.positions[t0 + r]));
   const int n_keys = (int)min((int64_t)a.context_lens[b], pmax + 1);
   const int kt_begin = (int)(lo_min / KT) * KT;  // (tiles stay aligned to absolute positions)
-  float m[4], l[4], acc[4][4];
+  float m[4], l[4], acc[4][NR];
   for (int i = 0; i < 4; i++) {
     m[i] = -INFINITY, l[i] = 0.f;
     if (a.sink) m[i] = a.sink[h], l[i] = 1.f;  // the sink: one more term exp(sink - m) of the denominator, present from the start
-    for (int r = 0; r < 4; r++) acc[i][r] = 0.f;
+    for (int r = 0; r < NR; r++) acc[i][r] = 0.f;
   }
   const T* kc = (const T*)a.kc;
   const T* vc = (const T*)a.vc;
@@ -594,11 +604,11 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
       }
       l[i] = l[i] * corr + wave_sum(p);
       m[i] = mn;
-      for (int rr = 0; rr < 4; rr++) acc[i][rr] *= corr;
+      for (int rr = 0; rr < NR; rr++) acc[i][rr] *= corr;
       if (lane < KT) ps[r * KT + lane] = p;
     }
     __syncthreads();
-    for (int rr = 0; rr < 4; rr++) {
+    for (int rr = 0; rr < NR; rr++) {
       const int d = lane + 64 * rr;
       if (d >= vdim) break;
 #pragma unroll 4
@@ -614,7 +624,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
     if (r >= nq) continue;
     float inv = l[i] > 0.f ? 1.f / l[i] : 0.f;
     if (a.gate) inv *= sigmoidf_(a.gate[(size_t)(t0 + r) * a.gate_ld + h]);
-    for (int rr = 0; rr < 4; rr++) {
+    for (int rr = 0; rr < NR; rr++) {
       const int d = lane + 64 * rr;
       if (d < vdim) El<T>::st(out + (size_t)(t0 + r) * a.H * vdim + h * vdim + d, acc[i][rr] * inv);
     }
@@ -844,7 +854,7 @@ __device__ __forceinline__ float stk_dot_row<uint16_t>(const float* qs, const ui
   for (int d = 0; d < dim; d++) d0 = fmaf(qs[d], BF16::to_f32(kr[d]), d0);
   return d0;
 }
-template <typename T>
+template <typename T, int NR>
 __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArgs a) {
   extern __shared__ float lds[];
   const int dim = a.dim, vdim = a.vdim;
@@ -865,7 +875,8 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
   const T* vc = (const T*)a.vc;
   const uint32_t* bt = a.block_tables + (size_t)b * a.max_blocks;
   const int kdim = a.k_ld ? a.k_ld : a.G * dim, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
-  float m = -INFINITY, l = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f, acc[NR];
+  for (int i = 0; i < NR; i++) acc[i] = 0.f;
   if (a.sink && wave == 0) m = a.sink[h], l = 1.f;
   // 16-bit values in whole octets: the value phase reads 16 bytes a lane (oc = channel octets rounded up to a power of two)
   const bool vec = sizeof(T) == 2 && vdim % 8 == 0 && vd_all % 8 == 0 && ((uintptr_t)vc % 16) == 0;
@@ -919,7 +930,7 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
           }
       }
     } else {
-      for (int rr = 0; rr < 4; rr++) {
+      for (int rr = 0; rr < NR; rr++) {
         const int d = lane + 64 * rr;
         if (d >= vdim) break;
         float o = acc[rr] * corr;
@@ -936,7 +947,7 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
     if (lane < oc && co * 8 < vdim)
       for (int i = 0; i < 8; i++) os[wave * vdim + co * 8 + i] = vacc[i];
   } else {
-    for (int rr = 0; rr < 4; rr++) {
+    for (int rr = 0; rr < NR; rr++) {
       const int d = lane + 64 * rr;
       if (d < vdim) os[wave * vdim + d] = acc[rr];
     }
@@ -973,19 +984,25 @@ void vra_stack_gemm(const StkGemmArgs& g, int dtype, int64_t stream) {
   const bool big = g.tile_group ? g.granule == 64 : g.M > 32;
   const bool mfma = dtype == VRA_BF16 && g.K % 8 == 0 && g.lda % 8 == 0 && ((uintptr_t)g.a % 16 == 0) && ((uintptr_t)g.w % 16 == 0) &&
                     (g.w_group_stride % 8 == 0) && (g.a_batch_stride % 8 == 0) && (g.w_batch_stride % 8 == 0);
-  VRA_CHECK_ARG(g.epi == 0 || (mfma && g.N % 32 == 0), "stack gemm: the gated epilogue needs the bf16 MFMA path and whole gate / up blocks");
+  VRA_CHECK_ARG(g.epi >= 0 && g.epi <= 2 && (g.epi != 2 || g.act == 3) && (g.softcap <= 0.f || g.epi != 1), "stack gemm: unknown epilogue");
+  const bool post = g.epi == 2 || g.softcap > 0.f;
+  VRA_CHECK_ARG(!post || !g.a_scale, "stack gemm: scaled rows and an element-wise epilogue do not come together");
+  VRA_CHECK_ARG(g.epi != 1 || (mfma && g.N % 32 == 0), "stack gemm: the gated epilogue needs the bf16 MFMA path and whole gate / up blocks");
   if (mfma) {
     if (big && !g.tile_group && !g.a_scale && g.M >= 256 && (int64_t)((g.M + 127) / 128) * ((g.N + 127) / 128) * nb >= 256) {
       // enough 128 x 128 tiles to fill the chip: a wave owns 64 x 64 (16 MFMAs per 8 fragment requests instead of 8 per 6)
       dim3 grid((g.M + 127) / 128, (g.N + 127) / 128, nb);
-      launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<4, 4, 2, 2, false><<<grid, 256, 0, st>>>(g); });
+      if (post) launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<4, 4, 2, 2, false, true><<<grid, 256, 0, st>>>(g); });
+      else launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<4, 4, 2, 2, false><<<grid, 256, 0, st>>>(g); });
     } else if (big) {
       dim3 grid((g.M + 63) / 64, (g.N + 127) / 128, nb);
       if (g.a_scale) launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<2, 4, 2, 2, true><<<grid, 256, 0, st>>>(g); });
+      else if (post) launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<2, 4, 2, 2, false, true><<<grid, 256, 0, st>>>(g); });
       else launch_checked("stack gemm", [&] { stk_gemm_mfma_kernel<2, 4, 2, 2, false><<<grid, 256, 0, st>>>(g); });
     } else {
       dim3 grid((g.M + 15) / 16, (g.N + 31) / 32, nb);
       if (g.a_scale) launch_checked("stack gemm", [&] { stk_gemm_mfma_small_kernel<true><<<grid, 512, 0, st>>>(g); });
+      else if (post) launch_checked("stack gemm", [&] { stk_gemm_mfma_small_kernel<false, true><<<grid, 512, 0, st>>>(g); });
       else launch_checked("stack gemm", [&] { stk_gemm_mfma_small_kernel<false><<<grid, 512, 0, st>>>(g); });
     }
     return;
@@ -1067,18 +1084,25 @@ void vra_stack_kv_store(const void* k, const void* v, int ld, void* kc, void* vc
 
 void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
   VRA_CHECK_ARG(a.q && a.out && a.kc && a.vc && a.positions && a.block_tables && a.context_lens, "stack attention: null pointer");
-  VRA_CHECK_ARG(a.B > 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.dim > 0 && a.vdim > 0 && a.vdim <= 256 && a.BS > 0 && a.max_blocks > 0,
-                "stack attention: heads must be a multiple of kv heads, value size at most 256");
+  VRA_CHECK_ARG(a.B > 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.dim > 0 && a.vdim > 0 && a.vdim <= 512 && a.BS > 0 && a.max_blocks > 0,
+                "stack attention: heads must be a multiple of kv heads, value size at most 512");
   hipStream_t st = as_stream(stream);
   if (!a.cu_q) {
     const size_t lds = ((size_t)a.dim + 2 * STK_DW * 64 + 2 * STK_DW + STK_DW * (size_t)a.vdim) * sizeof(float);
     VRA_CHECK_ARG(lds <= 64 * 1024, "stack attention: head does not fit LDS");
     dim3 grid(a.B, a.H);
-    if (dtype == VRA_F32) launch_checked("stack attention (decode)", [&] { stk_attn_decode_kernel<float><<<grid, 64 * STK_DW, lds, st>>>(a); });
-    else launch_checked("stack attention (decode)", [&] { stk_attn_decode_kernel<uint16_t><<<grid, 64 * STK_DW, lds, st>>>(a); });
+#define STK_DEC(TT, NRV) launch_checked("stack attention (decode)", [&] { stk_attn_decode_kernel<TT, NRV><<<grid, 64 * STK_DW, lds, st>>>(a); })
+    if (dtype == VRA_F32) {
+      if (a.vdim <= 256) STK_DEC(float, 4);
+      else STK_DEC(float, 8);
+    } else {
+      if (a.vdim <= 256) STK_DEC(uint16_t, 4);
+      else STK_DEC(uint16_t, 8);
+    }
+#undef STK_DEC
     return;
   }
-  if (dtype == VRA_BF16 && a.dim % 8 == 0 && a.vdim % 16 == 0 && a.dim <= 256 && a.ldq % 8 == 0 && ((uintptr_t)a.q % 16 == 0) && a.BS % 32 == 0 &&
+  if (dtype == VRA_BF16 && a.dim % 8 == 0 && a.vdim % 16 == 0 && a.dim <= 256 && a.vdim <= 256 && a.ldq % 8 == 0 && ((uintptr_t)a.q % 16 == 0) && a.BS % 32 == 0 &&
       a.k_ld % 8 == 0 && a.v_ld % 8 == 0 && ((uintptr_t)a.vc % 16 == 0)) {
     dim3 grid((a.max_q + 63) / 64, a.B, a.H);
 #define STK_PFM(DCV, VTV) launch_checked("stack attention (prefill, mfma)", [&] { stk_attn_prefill_mfma_kernel<DCV, VTV><<<grid, 256, 0, st>>>(a); })
@@ -1092,9 +1116,18 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
   auto need = [&](int kt) { return ((size_t)STK_QT * a.dim + (size_t)kt * (a.dim + 1) + (size_t)kt * a.vdim + (size_t)STK_QT * kt) * sizeof(float); };
   dim3 grid((a.max_q + STK_QT - 1) / STK_QT, a.B, a.H);
   const int kt = need(64) <= 64 * 1024 ? 64 : (need(32) <= 64 * 1024 ? 32 : 16);
-  VRA_CHECK_ARG(need(kt) <= 64 * 1024, "stack attention: head does not fit LDS");
   const size_t lds = need(kt);
-#define STK_PF(TT, KTV) launch_checked("stack attention (prefill)", [&] { stk_attn_prefill_kernel<TT, KTV><<<grid, 256, lds, st>>>(a); })
+  VRA_CHECK_ARG(lds <= 160 * 1024, "stack attention: head does not fit LDS");
+#define STK_PFN(TT, KTV, NRV)                                                                                                                     \
+  do {                                                                                                                                            \
+    if (lds > 64 * 1024) (void)hipFuncSetAttribute((const void*)stk_attn_prefill_kernel<TT, KTV, NRV>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+    launch_checked("stack attention (prefill)", [&] { stk_attn_prefill_kernel<TT, KTV, NRV><<<grid, 256, lds, st>>>(a); });                         \
+  } while (0)
+#define STK_PF(TT, KTV)                      \
+  do {                                       \
+    if (a.vdim <= 256) STK_PFN(TT, KTV, 4);  \
+    else STK_PFN(TT, KTV, 8);                \
+  } while (0)
   if (dtype == VRA_F32) {
     if (kt == 64) STK_PF(float, 64);
     else if (kt == 32) STK_PF(float, 32);
@@ -1105,6 +1138,7 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
     else STK_PF(uint16_t, 16);
   }
 #undef STK_PF
+#undef STK_PFN
 }
 
 // ================================================================================================ C entry points (one operator each)

@@ -68,6 +68,20 @@ __global__ __launch_bounds__(256) void stk_embed_pair_kernel(StkEmbedPairArgs a)
 }
 
 // ------------------------------------------------------------------------------------------------ seam of two sub-blocks (+ router)
+// takes the mean off a row whose elements every thread holds for itself (column c belongs to thread c mod 256) -> 1 / standard deviation
+__device__ __forceinline__ float center_rows(float* xs, int W, int tid, float eps, float* red) {
+  float s = 0.f;
+  for (int c = tid; c < W; c += 256) s += xs[c];
+  const float mean = block_sum_256(s, red) / (float)W;
+  s = 0.f;
+  for (int c = tid; c < W; c += 256) {
+    const float d = xs[c] - mean;
+    xs[c] = d;
+    s = fmaf(d, d, s);
+  }
+  return 1.f / sqrtf(block_sum_256(s, red) / (float)W + eps);
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   extern __shared__ float lds[];
@@ -118,7 +132,14 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
       xs[c] = v;
       s = fmaf(v, v, s);
     }
-    if (a.dyt) {
+    if (a.norm_kind == 2) {  // (two passes: the deviations are squared after the mean has been taken off)
+      const float r = center_rows(xs, W, tid, a.eps, red);
+      for (int c = tid; c < W; c += 256) {
+        const float v = x[c] + xs[c] * r * a.post_w[c];
+        x[c] = v;
+        xs[c] = v;
+      }
+    } else if (a.norm_kind == 1) {
       for (int c = tid; c < W; c += 256) {
         const float v = x[c] + (tanhf(a.post_alpha * xs[c]) * a.post_w[c] + a.post_b[c]);
         x[c] = v;
@@ -137,14 +158,16 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   }
   if (!a.pre_w) return;
   float r = 1.f;
-  if (!a.dyt) {
+  if (a.norm_kind == 2) {
+    r = center_rows(xs, W, tid, a.eps, red);
+  } else if (a.norm_kind == 0) {
     float s = 0.f;
     for (int c = tid; c < W; c += 256) s = fmaf(xs[c], xs[c], s);
     r = 1.f / sqrtf(block_sum_256(s, red) / (float)W + a.eps);
   }
   T* h = (T*)a.h + (size_t)t * W;
   for (int c = tid; c < W; c += 256) {
-    const float v = a.dyt ? tanhf(a.pre_alpha * xs[c]) * a.pre_w[c] + a.pre_b[c] : xs[c] * r * a.pre_w[c];
+    const float v = a.norm_kind == 1 ? tanhf(a.pre_alpha * xs[c]) * a.pre_w[c] + a.pre_b[c] : xs[c] * r * a.pre_w[c];
     xs[c] = v;
     El<T>::st(h + c, v);
     if (a.h32) a.h32[(size_t)t * W + c] = v;
@@ -213,7 +236,14 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   // over the lanes of wave 0 (their corrections are fetched side by side, not one after the other), the groups over the threads.
   float* sc = zs + n;        // [n] scores
   float* gs = zs + 2 * n;    // [n_groups]
-  if (wave == 0) {
+  const bool sig = a.router_kind == 2;
+  if (wave == 0 && sig) {
+    for (int e = lane; e < n; e += 64) {
+      const float sv = sigmoidf_(zs[e]);
+      sc[e] = sv;
+      zs[e] = sv + (a.router_bias ? a.router_bias[e] : 0.f);
+    }
+  } else if (wave == 0) {
     float m = -INFINITY, sum = 0.f;
     for (int e = lane; e < n; e += 64) m = fmaxf(m, zs[e]);
     m = wave_max(m);
@@ -233,9 +263,13 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   if (a.n_groups > 1 && a.keep < a.n_groups) {  // (uniform over the workgroup)
     const int per = n / a.n_groups;
     for (int g = tid; g < a.n_groups; g += 256) {
-      float b = zs[g * per];
-      for (int e = 1; e < per; e++) b = fmaxf(b, zs[g * per + e]);
-      gs[g] = b;
+      float b = zs[g * per], b2 = -INFINITY;  // the two largest
+      for (int e = 1; e < per; e++) {
+        const float v = zs[g * per + e];
+        b2 = fmaxf(b2, fminf(b, v));
+        b = fmaxf(b, v);
+      }
+      gs[g] = sig && per > 1 ? b + b2 : b;
     }
     __syncthreads();
     for (int g = tid; g < a.n_groups; g += 256) {  // a group stays if fewer than `keep` groups come before it (larger score, or equal and lower index)
@@ -252,7 +286,8 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
     const bool have = lane < n;
     const float val = have ? zs[lane] : 0.f, sv = have ? sc[lane] : 0.f;
     bool avail = have;
-    float idw = 0.f;
+    float idw = 0.f, sum = 0.f, pick_w = 0.f;
+    int pick_e = -1;  // (lane j keeps pick j: top <= n <= 64)
     for (int j = 0; j < a.top; j++) {
       const float v = avail ? val : -INFINITY;
       const float m = wave_max(v);
@@ -261,17 +296,20 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
       const float w = __shfl(sv, best, 64);
       if (lane == best) avail = false;
       const bool ident = best >= n_real;
-      if (lane == 0) {
-        a.pair_expert[(size_t)t * a.top + j] = ident ? -1 : best;
-        a.pair_weight[(size_t)t * a.top + j] = w;
-      }
+      if (lane == j) pick_e = ident ? -1 : best, pick_w = w;
       if (ident) idw += w;
+      sum += w;
     }
-    if (lane == 0 && a.id_weight) a.id_weight[t] = idw;
+    const float norm = sig ? sum + 1e-20f : 1.f;
+    if (lane < a.top) {
+      a.pair_expert[(size_t)t * a.top + lane] = pick_e;
+      a.pair_weight[(size_t)t * a.top + lane] = sig ? pick_w / norm : pick_w;
+    }
+    if (lane == 0 && a.id_weight) a.id_weight[t] = idw / norm;
     return;
   }
   if (tid != 0) return;
-  float idw = 0.f;
+  float idw = 0.f, sum = 0.f;
   for (int j = 0; j < a.top; j++) {
     int best = -1;
     float bz = -INFINITY;
@@ -283,8 +321,11 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
     a.pair_expert[(size_t)t * a.top + j] = ident ? -1 : best;
     a.pair_weight[(size_t)t * a.top + j] = w;
     if (ident) idw += w;
+    sum += w;
   }
-  if (a.id_weight) a.id_weight[t] = idw;
+  if (sig)
+    for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] /= sum + 1e-20f;
+  if (a.id_weight) a.id_weight[t] = sig ? idw / (sum + 1e-20f) : idw;
 }
 
 // ------------------------------------------------------------------------------------------------ per-head norm, rotary, cache rows
@@ -757,7 +798,8 @@ void vra_stack_embed_pair(const StkEmbedPairArgs& a, int dtype, int64_t stream) 
 void vra_stack_sandwich_norm(const StkSandwichArgs& a, int dtype, int64_t stream) {
   VRA_CHECK_ARG(a.x && a.T > 0 && a.W > 0 && (!a.post_w || (a.p1 && a.n1 >= 1)) && (!a.pre_w || a.h), "stack seam norm: null pointer or empty shape");
   VRA_CHECK_ARG(!a.router_w || (a.pre_w && a.pair_expert && a.pair_weight && a.top >= 1 && a.top <= a.n_router), "stack seam norm: router outputs");
-  VRA_CHECK_ARG(!a.dyt || ((!a.post_w || a.post_b) && (!a.pre_w || a.pre_b)), "stack seam norm: Dynamic Tanh needs its offsets");
+  VRA_CHECK_ARG(a.norm_kind >= 0 && a.norm_kind <= 2 && a.router_kind >= 0 && a.router_kind <= 2, "stack seam norm: unknown norm or router kind");
+  VRA_CHECK_ARG(a.norm_kind != 1 || ((!a.post_w || a.post_b) && (!a.pre_w || a.pre_b)), "stack seam norm: Dynamic Tanh needs its offsets");
   VRA_CHECK_ARG((!a.p1_norm_w && !a.p2_norm_w) || a.n1 == 1, "stack seam norm: a part with a norm of its own is one row a token");
   VRA_CHECK_ARG(a.router_kind == 0 || !a.router_w ||
                     (a.n_identity >= 0 && a.n_identity < a.n_router && (a.n_groups <= 1 || (a.n_router % a.n_groups == 0 && a.keep >= 1)) &&
@@ -920,14 +962,14 @@ extern "C" void vra_stack_op_attention_window(const void* q, int32_t ldq, void* 
 }
 // the seam with Dynamic Tanh norms, per-branch norms, pairs without a row, a weighted second part and the router over all outputs
 extern "C" void vra_stack_op_seam(float* x, const float* p1, int32_t n1, const float* pw, const int32_t* pe, float c1, const float* p2, const float* p2w,
-                                  float c2, const float* p1_norm_w, const float* p2_norm_w, int32_t dyt, const float* post_w, const float* post_b,
+                                  float c2, const float* p1_norm_w, const float* p2_norm_w, int32_t norm_kind, const float* post_w, const float* post_b,
                                   float post_alpha, const float* pre_w, const float* pre_b, float pre_alpha, void* h, float* h32, float eps, int32_t T,
                                   int32_t W, const void* router_w, const float* router_bias, int32_t router_kind, int32_t n_router, int32_t top,
                                   int32_t n_groups, int32_t keep, int32_t n_identity, int32_t* pair_expert, float* pair_weight, float* id_weight,
                                   int32_t dtype, int64_t stream) {
   StkSandwichArgs a;
   a.x = x, a.p1 = p1, a.n1 = n1, a.pw = pw, a.pe = pe, a.c1 = c1, a.p2 = p2, a.p2w = p2w, a.c2 = c2, a.p1_norm_w = p1_norm_w, a.p2_norm_w = p2_norm_w;
-  a.dyt = dyt, a.post_w = post_w, a.post_b = post_b, a.post_alpha = post_alpha, a.pre_w = pre_w, a.pre_b = pre_b, a.pre_alpha = pre_alpha;
+  a.norm_kind = norm_kind, a.post_w = post_w, a.post_b = post_b, a.post_alpha = post_alpha, a.pre_w = pre_w, a.pre_b = pre_b, a.pre_alpha = pre_alpha;
   a.h = h, a.h32 = h32, a.eps = eps, a.T = T, a.W = W, a.router_w = router_w, a.router_bias = router_bias, a.router_kind = router_kind;
   a.n_router = n_router, a.top = top, a.n_groups = n_groups, a.keep = keep, a.n_identity = n_identity;
   a.pair_expert = pair_expert, a.pair_weight = pair_weight, a.id_weight = id_weight;

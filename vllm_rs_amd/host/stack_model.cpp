@@ -66,11 +66,11 @@ bool StackModel::parse_spec(const char* spec) {
         *out = v == b ? 1 : (c && v == c ? 2 : 0);
         return true;
       };
-      if (!pick("block", "parallel", "sequential", &block_, "sandwich") || !pick("norm", "rms", "dyt", &norm_kind_) || !pick("pos", "sinusoid", "none", &pos_kind_))
+      if (!pick("block", "parallel", "sequential", &block_, "sandwich") || !pick("norm", "rms", "dyt", &norm_kind_, "layer") || !pick("pos", "sinusoid", "none", &pos_kind_))
         return false;
       norm_offset_ = (float)num("norm_offset", 0.0), embed_scale_ = (float)num("embed_scale", 1.0), embed_norm_ = (int)num("embed_norm", 0);
       pair_buckets_ = (int)num("pair_buckets", 0), pair_mul_prev_ = (int64_t)num("pair_mul_prev", 0), pair_mul_cur_ = (int64_t)num("pair_mul_cur", 0);
-      tie_head_ = (int)num("tie_head", 0);
+      tie_head_ = (int)num("tie_head", 0), layer_scale_ = (int)num("layer_scale", 0), logit_softcap_ = (float)num("logit_softcap", 0.0);
     } else if (kind == "layer") {
       StackLayer L;
       L.heads = (int)num("heads", 0), L.kv_heads = (int)num("kv_heads", L.heads), L.dim = (int)num("dim", 0), L.vdim = (int)num("vdim", L.dim);
@@ -91,13 +91,13 @@ bool StackModel::parse_spec(const char* spec) {
       }
       {
         const std::string rk = f.count("router") ? f["router"] : "sigmoid", ak = f.count("act") ? f["act"] : "clamped";
-        if ((rk != "sigmoid" && rk != "softmax" && rk != "softmax_all") || (ak != "clamped" && ak != "silu"))
-          return spec_error_ = "layer stack spec: router is sigmoid or softmax or softmax_all, act clamped or silu", false;
-        L.router_kind = rk == "softmax" ? 1 : (rk == "softmax_all" ? 2 : 0), L.act_kind = ak == "silu" ? 2 : 0;
+        if ((rk != "sigmoid" && rk != "softmax" && rk != "softmax_all" && rk != "sigmoid_norm") || (ak != "clamped" && ak != "silu" && ak != "gelu"))
+          return spec_error_ = "layer stack spec: router is sigmoid or softmax or softmax_all or sigmoid_norm, act clamped or silu or gelu", false;
+        L.router_kind = rk == "softmax" ? 1 : (rk == "softmax_all" ? 2 : (rk == "sigmoid_norm" ? 3 : 0)), L.act_kind = ak == "silu" ? 2 : (ak == "gelu" ? 3 : 0);
         L.n_identity = (int)num("identity", 0), L.n_groups = (int)num("groups", 0), L.keep = (int)num("keep", 0);
       }
       {
-        const std::string rt = f.count("right") ? f["right"] : "gla", rl = f.count("rot_layout") ? f["rot_layout"] : "half";
+        const std::string rt = f.count("right") ? f["right"] : "gla", rl = f.count("rot_layout") ? f["rot_layout"] : (L.mixer == 1 ? "pairs" : "half");
         if ((rt != "gla" && rt != "rglru") || (rl != "half" && rl != "pairs")) return spec_error_ = "layer stack spec: right is gla or rglru, rot_layout half or pairs", false;
         L.right_kind = rt == "rglru", L.rot_layout = rl == "pairs";
         L.lowrank = (int)num("lowrank", 1), L.r_width = (int)num("r_width", 0), L.r_blocks = (int)num("r_blocks", 1);
@@ -120,6 +120,8 @@ bool StackModel::parse_spec(const char* spec) {
     }
   }
   if (!have_stack || width_ <= 0 || vocab_ <= 0 || layers_.empty()) return spec_error_ = "layer stack spec: width, vocab and at least one layer are needed", false;
+  if (norm_kind_ == 2 && block_ != 2) return spec_error_ = "layer stack spec: layer norms belong to sandwich blocks", false;
+  if (layer_scale_ && (block_ != 2 || norm_kind_ == 1)) return spec_error_ = "layer stack spec: layer_scale belongs to sandwich blocks with rms or layer norms", false;
   if (groups_ < 1 || width_ % groups_) return spec_error_ = "layer stack spec: the width must split into equal norm groups", false;
   if (width_ != mc_.hidden_size || vocab_ != mc_.vocab_size || (int)layers_.size() != mc_.num_layers)
     return spec_error_ = "layer stack spec: width / vocab / layers differ from the model config", false;
@@ -128,11 +130,13 @@ bool StackModel::parse_spec(const char* spec) {
     const std::string at = " (layer " + std::to_string(i) + ")";
     if (L.heads <= 0 || L.kv_heads <= 0 || L.heads % L.kv_heads || L.dim <= 0 || L.vdim <= 0 || (L.mixer == 0 && L.vdim > 256))
       return spec_error_ = "layer stack spec: heads must be a multiple of kv_heads, sizes positive, value size at most 256" + at, false;
-    if ((L.mixer == 1 || L.mixer == 2) && block_ != 1) return spec_error_ = "layer stack spec: latent and sigmoid mixers run in sequential blocks" + at, false;
+    if ((L.mixer == 2 && block_ != 1) || (L.mixer == 1 && block_ == 0))
+      return spec_error_ = "layer stack spec: latent and sigmoid mixers run in sequential blocks, the latent one also in sandwich blocks" + at, false;
     if (L.mixer == 0 && block_ != 0) return spec_error_ = "layer stack spec: the softmax mixer with temperature and cap runs in parallel blocks" + at, false;
     if (L.mixer >= 3 && block_ != 2) return spec_error_ = "layer stack spec: delta, retention and parallel mixers run in sandwich blocks" + at, false;
-    if (block_ == 2 && (L.mixer < 3 || (L.mlp != 0 && L.mlp != 2 && L.mlp != 4) || L.weights_of >= 0))
-      return spec_error_ = "layer stack spec: sandwich blocks hold delta, retention, lightning or parallel mixers and a mixture of experts, a clamped dense feed-forward or none" + at, false;
+    if (block_ == 2 && ((L.mixer < 3 && L.mixer != 1) || (L.mlp != 0 && L.mlp != 2 && L.mlp != 4)))
+      return spec_error_ = "layer stack spec: sandwich blocks hold latent, delta, retention, lightning or parallel mixers and a mixture of experts, a clamped dense feed-forward or none" + at, false;
+    if (block_ == 2 && L.weights_of >= 0 && L.mixer != 1) return spec_error_ = "layer stack spec: in sandwich blocks only layers with the latent mixer share weights" + at, false;
     if (L.mlp == 4 && block_ != 2) return spec_error_ = "layer stack spec: the clamped dense feed-forward belongs to sandwich blocks" + at, false;
     if (L.mixer == 3 && (L.conv < 1 || (L.lowrank && (L.rank_a < 1 || L.rank_g < 1)) || L.dim > 256)) return spec_error_ = "layer stack spec: the delta mixer needs conv >= 1, rank_a, rank_g, dim <= 256" + at, false;
     if (L.mixer == 6 && ((int)L.decay.size() != L.heads || L.kv_heads != L.heads || L.dim > 256))
@@ -141,9 +145,11 @@ bool StackModel::parse_spec(const char* spec) {
         (L.r_width <= 0 || L.r_blocks < 1 || L.r_width % L.r_blocks || L.conv < 1 || L.rot_dims < 0 || L.rot_dims > L.dim || L.rot_dims % 2 || L.chunk < 0 ||
          L.window < 0 || L.vdim > 256 || (L.yarn_factor > 0.0 && (L.yarn_original <= 0.0 || L.yarn_fast <= 0.0 || L.yarn_slow <= 0.0))))
       return spec_error_ = "layer stack spec: the parallel mixer with a gated recurrence needs r_width in r_blocks equal blocks, r_conv >= 1, an even rot_dims <= dim, vdim <= 256" + at, false;
-    if ((L.window > 0 || L.head_temp || L.head_gate || L.rot_layout || L.branch_norm) && L.mixer != 5 && L.mixer != 2)
-      return spec_error_ = "layer stack spec: window, head_temp, head_gate, rot_layout and branch_norm belong to the parallel mixer" + at, false;
-    if (L.router_kind == 2 && (L.n_identity < 0 ||
+    if (((L.window > 0 || L.head_gate || L.rot_layout) && L.mixer != 5 && L.mixer != 2 && L.mixer != 1) || ((L.head_temp || L.branch_norm) && L.mixer != 5 && L.mixer != 2))
+      return spec_error_ = "layer stack spec: window, head_temp, head_gate, rot_layout and branch_norm belong to the parallel mixer (the first, third and fourth also to the latent one)" + at, false;
+    if (L.router_kind == 3 && L.n_identity) return spec_error_ = "layer stack spec: identity experts belong to router=softmax_all" + at, false;
+    if (L.act_kind == 3 && (L.mlp != 2 || L.router_kind != 3)) return spec_error_ = "layer stack spec: experts without a gate belong to router=sigmoid_norm" + at, false;
+    if (L.router_kind >= 2 && (L.n_identity < 0 ||
                                (L.n_groups > 1 && ((L.experts + L.n_identity) % L.n_groups || L.keep < 1 || L.keep > L.n_groups))))
       return spec_error_ = "layer stack spec: router groups must divide experts + identity, 1 <= keep <= groups" + at, false;
     if (L.mixer == 4 && ((int)L.decay.size() != L.heads || L.kv_heads != L.heads || L.rot_dims < 0 || L.rot_dims > L.dim || L.rot_dims % 2 || L.dim > 256))
@@ -151,11 +157,12 @@ bool StackModel::parse_spec(const char* spec) {
     if (L.mixer == 5 && L.right_kind == 0 && (L.r_heads <= 0 || L.r_dim <= 0 || L.r_dim > 256 || L.r_vdim <= 0 || L.rank_a < 1 || !(L.tau > 0.f) || L.rot_dims < 0 || L.rot_dims > L.dim || L.rot_dims % 2 ||
                          L.chunk < 0 || L.vdim > 256 || (L.rs_factor > 0.0 && (L.rs_original <= 0.0 || L.rs_high <= L.rs_low))))
       return spec_error_ = "layer stack spec: the parallel mixer needs r_heads, r_dim <= 256, r_vdim, rank_a, tau > 0, an even rot_dims <= dim, vdim <= 256" + at, false;
-    if (L.router_kind >= 1 && (block_ != 2 || L.shared_ff > 0)) return spec_error_ = "layer stack spec: the softmax router belongs to sandwich blocks and has no shared expert" + at, false;
+    if (L.router_kind == 3 && block_ != 2) return spec_error_ = "layer stack spec: the normalised sigmoid router belongs to sandwich blocks" + at, false;
+    if ((L.router_kind == 1 || L.router_kind == 2) && (block_ != 2 || L.shared_ff > 0)) return spec_error_ = "layer stack spec: the softmax router belongs to sandwich blocks and has no shared expert" + at, false;
     if (L.mixer != 0 && L.kv_from >= 0) return spec_error_ = "layer stack spec: kv_from belongs to the softmax mixer" + at, false;
-    if (L.mixer == 1 && (L.kv_rank <= 0 || L.q_rank <= 0 || L.rot_dim < 0 || L.kv_rank > 256 || L.rot_dims < 0 || L.rot_dims > L.rot_dim || L.rot_dims % 2 ||
+    if (L.mixer == 1 && (L.kv_rank <= 0 || L.q_rank <= 0 || L.rot_dim < 0 || L.kv_rank > 512 || L.rot_dims < 0 || L.rot_dims > L.rot_dim || L.rot_dims % 2 ||
                          (L.yarn_factor > 0.0 && (L.yarn_original <= 0.0 || L.yarn_fast <= 0.0 || L.yarn_slow <= 0.0))))
-      return spec_error_ = "layer stack spec: latent attention needs q_rank, 0 < kv_rank <= 256, an even rot_dims <= rot_dim" + at, false;
+      return spec_error_ = "layer stack spec: latent attention needs q_rank, 0 < kv_rank <= 512, an even rot_dims <= rot_dim" + at, false;
     if ((L.mlp == 3) != (block_ == 1) && L.mlp != 0) return spec_error_ = "layer stack spec: the gated feed-forward belongs to sequential blocks, the others to parallel ones" + at, false;
     if (L.weights_of >= 0) {
       int root = L.weights_of;  // (a chain of references ends at a layer with tensors of its own)
@@ -165,7 +172,7 @@ bool StackModel::parse_spec(const char* spec) {
       L.weights_of = root;
       const StackLayer& S = layers_[root];
       if (S.mixer != L.mixer || S.heads != L.heads || S.kv_heads != L.kv_heads || S.dim != L.dim || S.vdim != L.vdim || S.rot_dim != L.rot_dim ||
-          S.kv_rank != L.kv_rank || S.q_rank != L.q_rank || S.mlp != L.mlp || S.ff != L.ff || S.kv_from >= 0 || L.kv_from >= 0)
+          S.kv_rank != L.kv_rank || S.q_rank != L.q_rank || S.window != L.window || S.head_gate != L.head_gate || S.experts != L.experts || S.shared_ff != L.shared_ff || S.mlp != L.mlp || S.ff != L.ff || S.kv_from >= 0 || L.kv_from >= 0)
         return spec_error_ = "layer stack spec: a layer that shares weights has the shapes of the layer it names" + at, false;
     }
     if (!L.has_cache()) {
@@ -338,6 +345,17 @@ bool StackModel::finalize_weights() {
     for (float& e : v) e += norm_offset_;
     return (*w = upload_floats(v)) != nullptr;
   };
+  // the norm of a sub-block's output with the layer's scale: one factor per channel, folded into the norm's weight in f32 (two bf16 values'
+  // product is exact there)
+  auto up_norm_scaled = [&](const std::string& name, const std::string& scale, float** w) {
+    if (!layer_scale_) return up_norm_off(name, W, w);
+    const HostTensor *t, *s;
+    if (!need(name, W, -1, &t) || !need(scale, W, -1, &s)) return false;
+    std::vector<float> v, f;
+    f32_of(*t, &v), f32_of(*s, &f);
+    for (int i = 0; i < W; i++) v[i] = (v[i] + norm_offset_) * f[i];
+    return (*w = upload_floats(v)) != nullptr;
+  };
   // the shape a staged tensor came with (sizes the config does not carry: the ranks of low-rank projections)
   auto rows_of = [&](const std::string& name, int64_t cols) -> int64_t {
     auto it = staged_.find(name);
@@ -364,8 +382,8 @@ bool StackModel::finalize_weights() {
       if (!up_norm(p + "norm1", &L.norm_w, &L.norm_b, &L.norm_alpha) || !up_norm(p + "norm1b", &L.post1_w, &L.post1_b, &L.post1_alpha)) return false;
       if (L.mlp != 0 && (!up_norm(p + "norm2", &L.norm2_w, &L.norm2_b, &L.norm2_alpha) || !up_norm(p + "norm2b", &L.post2_w, &L.post2_b, &L.post2_alpha))) return false;
     } else if (block_ == 2) {
-      if (!up_norm_off(p + "norm1", W, &L.norm_w) || !up_norm_off(p + "norm1b", W, &L.post1_w)) return false;
-      if (L.mlp != 0 && (!up_norm_off(p + "norm2", W, &L.norm2_w) || !up_norm_off(p + "norm2b", W, &L.post2_w))) return false;
+      if (!up_norm_off(p + "norm1", W, &L.norm_w) || !up_norm_scaled(p + "norm1b", p + "ls1", &L.post1_w)) return false;
+      if (L.mlp != 0 && (!up_norm_off(p + "norm2", W, &L.norm2_w) || !up_norm_scaled(p + "norm2b", p + "ls2", &L.post2_w))) return false;
     } else {
       if (!up_norm(p + "norm1", &L.norm_w, &L.norm_b, &L.norm_alpha)) return false;
       if (block_ == 1 && L.mlp != 0 && !up_norm(p + "norm2", &L.norm2_w, &L.norm2_b, &L.norm2_alpha)) return false;
@@ -528,12 +546,13 @@ bool StackModel::finalize_weights() {
       if (k) parts.push_back(k), parts.push_back(v);
       if (!up_rows(parts, &L.qkv)) return false;
     } else if (L.mixer == 1) {
-      // the two down-projections in one matrix [q latent | kv latent | rotated key part]; W_uk per head transposed, so that a query is
+      // the two down-projections in one matrix [q latent | kv latent | rotated key part (| head gates)]; W_uk per head transposed, so that a query is
       // carried into the latent's space (q_h . (W_uk_h c) = (W_uk_h^T q_h) . c) and the cache needs the latent alone
-      const HostTensor *dq, *dkv, *uk;
+      const HostTensor *dq, *dkv, *uk, *hg = nullptr;
       const int H = L.heads, qd = L.dim + L.rot_dim;
       if (!need(p + "mix.dq", L.q_rank, W, &dq) || !need(p + "mix.dkv", L.kv_rank + L.rot_dim, W, &dkv) || !matrix(dq) || !matrix(dkv)) return false;
-      if (!up_rows({dq, dkv}, &L.qkv)) return false;
+      if (L.head_gate && (!need(p + "mix.g", H, W, &hg) || !matrix(hg))) return false;
+      if (!up_rows(hg ? std::vector<const HostTensor*>{dq, dkv, hg} : std::vector<const HostTensor*>{dq, dkv}, &L.qkv)) return false;
       if (!up_vec(p + "mix.dq.norm", L.q_rank, &L.qn_w) || !up_vec(p + "mix.dkv.norm", L.kv_rank, &L.kn_w)) return false;
       if (!up_mat(p + "mix.uq", (int64_t)H * qd, L.q_rank, &L.uq) || !up_mat(p + "mix.uv", (int64_t)H * L.vdim, L.kv_rank, &L.uv)) return false;
       if (!need(p + "mix.uk", (int64_t)H * L.dim, L.kv_rank, &uk) || !matrix(uk)) return false;
@@ -545,26 +564,8 @@ bool StackModel::finalize_weights() {
       weight_bytes_ += tr.size();
       if (!(L.ukt = upload(tr.data(), tr.size()))) return false;
       if (L.sink && !up_vec(p + "mix.sink", H, &L.sink_w)) return false;
-      // rotary frequencies in f64, kept as hi + lo f32 pairs
-      L.rot_pairs = L.rot_dims / 2;
-      std::vector<float> fh(std::max(L.rot_pairs, 1)), fl(std::max(L.rot_pairs, 1));
-      const double dims = (double)L.rot_dims, lnb = log(L.rot_base);
-      double lo = 0.0, hi = 0.0;
-      L.rot_mag = 1.f;
-      if (L.yarn_factor > 0.0) {
-        auto turn_dim = [&](double turns) { return dims * log(L.yarn_original / (2.0 * M_PI * turns)) / (2.0 * lnb); };
-        lo = std::max(floor(turn_dim(L.yarn_fast)), 0.0), hi = std::min(ceil(turn_dim(L.yarn_slow)), dims - 1.0);
-        L.rot_mag = (float)(0.1 * log(L.yarn_factor) + 1.0);
-      }
-      for (int i = 0; i < L.rot_pairs; i++) {
-        double fr = pow(L.rot_base, -2.0 * (double)i / dims);
-        if (L.yarn_factor > 0.0) {
-          const double ramp = std::min(std::max(((double)i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
-          fr = fr / L.yarn_factor * ramp + fr * (1.0 - ramp);
-        }
-        fh[i] = (float)fr, fl[i] = (float)(fr - (double)fh[i]);
-      }
-      if (!(L.freq_hi = upload_floats(fh)) || !(L.freq_lo = upload_floats(fl))) return false;
+      rotary_table(L);
+      if (!L.freq_hi || !L.freq_lo) return false;
     } else {
       // q | k | v | output gate in one matrix, the biases of q, k, v as one f32 row (zeros under the gate)
       const HostTensor *q, *k, *v, *g, *qb, *kb, *vb, *tk;
@@ -601,31 +602,33 @@ bool StackModel::finalize_weights() {
     } else if (L.mlp == 2) {
       const HostTensor *r, *sg = nullptr;
       if (!need(p + "mlp.router", L.experts + L.n_identity, W, &r) || !matrix(r)) return false;
-      if (L.shared_ff > 0 && (!need(p + "mlp.shared.sg", W, -1, &sg) || !matrix(sg))) return false;
+      if (L.shared_ff > 0 && L.router_kind == 0 && (!need(p + "mlp.shared.sg", W, -1, &sg) || !matrix(sg))) return false;
       std::vector<uint8_t> rt(r->data);
       if (sg) rt.insert(rt.end(), sg->data.begin(), sg->data.end());
       weight_bytes_ += rt.size();
       if (!(L.router = upload(rt.data(), rt.size()))) return false;
       if (L.router_kind == 1 && !up_vec(p + "mlp.router.b", L.experts, &L.router_bias)) return false;
-      if (L.router_kind == 2 && !up_vec(p + "mlp.correction", L.experts + L.n_identity, &L.router_bias)) return false;
-      std::vector<uint8_t> gu((size_t)L.experts * 2 * L.ffp * W * es), dn((size_t)L.experts * W * L.ffp * es);
+      if (L.router_kind >= 2 && !up_vec(p + "mlp.correction", L.experts + L.n_identity, &L.router_bias)) return false;
+      const size_t halves = L.gated() ? 2 : 1;
+      std::vector<uint8_t> gu((size_t)L.experts * halves * L.ffp * W * es), dn((size_t)L.experts * W * L.ffp * es);
       for (int e = 0; e < L.experts; e++) {
         const std::string pe = p + "mlp.e" + std::to_string(e) + ".";
-        const HostTensor *g, *u, *d;
-        if (!need(pe + "gate", L.ff, W, &g) || !need(pe + "up", L.ff, W, &u) || !need(pe + "down", W, L.ff, &d) || !matrix(g) || !matrix(u) || !matrix(d))
-          return false;
-        interleave(g, u, L.ff, L.ffp, gu.data() + (size_t)e * 2 * L.ffp * W * es);
+        const HostTensor *g = nullptr, *u, *d;
+        if (L.gated() && (!need(pe + "gate", L.ff, W, &g) || !matrix(g))) return false;
+        if (!need(pe + "up", L.ff, W, &u) || !need(pe + "down", W, L.ff, &d) || !matrix(u) || !matrix(d)) return false;
+        if (g) interleave(g, u, L.ff, L.ffp, gu.data() + (size_t)e * 2 * L.ffp * W * es);
+        else memcpy(gu.data() + (size_t)e * L.ffp * W * es, u->data.data(), u->data.size());  // (the rows beyond ff stay zero)
         pad_cols(d, L.ff, L.ffp, dn.data() + (size_t)e * W * L.ffp * es);
       }
       weight_bytes_ += gu.size() + dn.size();
       if (!(L.e_gu = upload(gu.data(), gu.size())) || !(L.e_down = upload(dn.data(), dn.size()))) return false;
       if (L.shared_ff > 0) {
-        const HostTensor *g, *u, *d;
-        if (!need(p + "mlp.shared.gate", L.shared_ff, W, &g) || !need(p + "mlp.shared.up", L.shared_ff, W, &u) ||
-            !need(p + "mlp.shared.down", W, L.shared_ff, &d) || !matrix(g) || !matrix(u) || !matrix(d))
-          return false;
-        std::vector<uint8_t> sgu((size_t)2 * L.sffp * W * es), sdn((size_t)W * L.sffp * es);
-        interleave(g, u, L.shared_ff, L.sffp, sgu.data());
+        const HostTensor *g = nullptr, *u, *d;
+        if (L.gated() && (!need(p + "mlp.shared.gate", L.shared_ff, W, &g) || !matrix(g))) return false;
+        if (!need(p + "mlp.shared.up", L.shared_ff, W, &u) || !need(p + "mlp.shared.down", W, L.shared_ff, &d) || !matrix(u) || !matrix(d)) return false;
+        std::vector<uint8_t> sgu(halves * L.sffp * W * es), sdn((size_t)W * L.sffp * es);
+        if (g) interleave(g, u, L.shared_ff, L.sffp, sgu.data());
+        else memcpy(sgu.data(), u->data.data(), u->data.size());
         pad_cols(d, L.shared_ff, L.sffp, sdn.data());
         weight_bytes_ += sgu.size() + sdn.size();
         if (!(L.s_gu = upload(sgu.data(), sgu.size())) || !(L.s_down = upload(sdn.data(), sdn.size()))) return false;
@@ -679,15 +682,16 @@ bool StackModel::init_synthetic(uint64_t seed) {
   const int W = width_;
   put("embed", vocab_, W, 0, 1.0);
   if (!tie_head_) put("head", vocab_, W, 0, 1.0 / sqrt((double)W));
+  const double around = 1.0 - (double)norm_offset_;
   auto put_norm = [&](const std::string& name) {
     put(name, W, 0, 1, 0.05);
     if (norm_kind_ == 1) put(name + ".b", W, 0, 0, 0.02), put(name + ".alpha", 1, 0, 0.5, 0.0);
   };
   if (block_ == 2 && norm_kind_ == 1) {
     put_norm("final.norm");
-  } else if (block_ == 2) {  // norm weights are stored around zero; the embedding's own norm and the token-pair table
-    put("final.norm", W, 0, 0, 0.05);
-    if (embed_norm_) put("embed.norm", W, 0, 0, 0.05);
+  } else if (block_ == 2) {  // norm weights are stored around 1 - norm_offset; the embedding's own norm and the token-pair table
+    put("final.norm", W, 0, around, 0.05);
+    if (embed_norm_) put("embed.norm", W, 0, around, 0.05);
     if (pair_buckets_ > 0) put("bigram", (int64_t)pair_buckets_ + 1, W, 0, 1.0);
   } else {
     put_norm("final.norm");
@@ -701,8 +705,10 @@ bool StackModel::init_synthetic(uint64_t seed) {
       put_norm(p + "norm1"), put_norm(p + "norm1b");
       if (L.mlp != 0) put_norm(p + "norm2"), put_norm(p + "norm2b");
     } else if (block_ == 2) {
-      put(p + "norm1", W, 0, 0, 0.05), put(p + "norm1b", W, 0, 0, 0.05);
-      if (L.mlp != 0) put(p + "norm2", W, 0, 0, 0.05), put(p + "norm2b", W, 0, 0, 0.05);
+      put(p + "norm1", W, 0, around, 0.05), put(p + "norm1b", W, 0, around, 0.05);
+      if (L.mlp != 0) put(p + "norm2", W, 0, around, 0.05), put(p + "norm2b", W, 0, around, 0.05);
+      if (layer_scale_) put(p + "ls1", W, 0, 0.8, 0.1);
+      if (layer_scale_ && L.mlp != 0) put(p + "ls2", W, 0, 0.8, 0.1);
     } else {
       put_norm(p + "norm1");
       if (block_ == 1 && L.mlp != 0) put_norm(p + "norm2");
@@ -767,6 +773,7 @@ bool StackModel::init_synthetic(uint64_t seed) {
       put(p + "mix.uk", (int64_t)L.heads * L.dim, L.kv_rank, 0, 1.0 / sqrt((double)L.kv_rank));
       put(p + "mix.uv", (int64_t)L.heads * L.vdim, L.kv_rank, 0, 1.0 / sqrt((double)L.kv_rank));
       if (L.sink) put(p + "mix.sink", L.heads, 0, 0, 1.0);
+      if (L.head_gate) put(p + "mix.g", L.heads, W, 0, sw);
     } else {
       put(p + "mix.q", L.nq(), W, 0, sw), put(p + "mix.k", L.nk(), W, 0, sw), put(p + "mix.v", L.nv(), W, 0, sw);
       put(p + "mix.g", (int64_t)L.heads * L.vdim, W, 0, sw);
@@ -787,14 +794,16 @@ bool StackModel::init_synthetic(uint64_t seed) {
     } else if (L.mlp == 2) {
       put(p + "mlp.router", L.experts + L.n_identity, W, 0, sw);
       if (L.router_kind == 1) put(p + "mlp.router.b", L.experts, 0, 0, 0.1);
-      if (L.router_kind == 2) put(p + "mlp.correction", L.experts + L.n_identity, 0, 0, 0.02);
+      if (L.router_kind >= 2) put(p + "mlp.correction", L.experts + L.n_identity, 0, 0, 0.02);
       for (int e = 0; e < L.experts; e++) {
         const std::string pe = p + "mlp.e" + std::to_string(e) + ".";
-        put(pe + "gate", L.ff, W, 0, sw), put(pe + "up", L.ff, W, 0, sw), put(pe + "down", W, L.ff, 0, 1.0 / sqrt((double)L.ff));
+        if (L.gated()) put(pe + "gate", L.ff, W, 0, sw);
+        put(pe + "up", L.ff, W, 0, sw), put(pe + "down", W, L.ff, 0, 1.0 / sqrt((double)L.ff));
       }
       if (L.shared_ff > 0) {
-        put(p + "mlp.shared.gate", L.shared_ff, W, 0, sw), put(p + "mlp.shared.up", L.shared_ff, W, 0, sw);
-        put(p + "mlp.shared.down", W, L.shared_ff, 0, 1.0 / sqrt((double)L.shared_ff)), put(p + "mlp.shared.sg", 1, W, 0, sw);
+        if (L.gated()) put(p + "mlp.shared.gate", L.shared_ff, W, 0, sw);
+        if (L.router_kind == 0) put(p + "mlp.shared.sg", 1, W, 0, sw);
+        put(p + "mlp.shared.up", L.shared_ff, W, 0, sw), put(p + "mlp.shared.down", W, L.shared_ff, 0, 1.0 / sqrt((double)L.shared_ff));
       }
     }
   }
@@ -975,11 +984,14 @@ bool StackModel::expert_pair(const void* a, int lda, const void* w_gu, int64_t g
                              float* out, int64_t stream, int act) {
   const int W = width_;
   StkGemmArgs g;
-  g.a = a, g.lda = lda, g.w = w_gu, g.w_group_stride = gu_stride, g.M = rows, g.N = 2 * fp, g.K = W;
+  g.a = a, g.lda = lda, g.w = w_gu, g.w_group_stride = gu_stride, g.M = rows, g.N = (act == 3 ? 1 : 2) * fp, g.K = W;
   g.tile_group = tile_group, g.granule = granule, g.a_row = a_row, g.a_scale = a_scale;
   g.limit = limit, g.act = act;
   const bool fused = dt_ == VRA_BF16 && W % 8 == 0 && lda % 8 == 0;
-  if (fused) {
+  if (act == 3) {  // no gate: an element-wise activation, in the epilogue whatever the type
+    g.epi = 2, g.out = act_, g.ldo = fp;
+    vra_stack_gemm(g, dt_, stream);
+  } else if (fused) {
     g.epi = 1, g.out = act_, g.ldo = fp;
     vra_stack_gemm(g, dt_, stream);
   } else {
@@ -1078,7 +1090,7 @@ bool StackModel::mixer_latent(const StackLayer& L, const InputMetadata& md, int6
   StkLatentPrepArgs lp;
   lp.raw = z_, lp.ld = L.nqkv(), lp.q_rank = L.q_rank, lp.kv_rank = L.kv_rank, lp.rot_dim = L.rot_dim, lp.qn_w = L.qn_w, lp.kvn_w = L.kn_w, lp.eps = eps_;
   lp.cq = act_, lp.cache = kc_[L.cache], lp.cache_ld = kd, lp.slots = md.slot_mapping, lp.positions = md.positions, lp.T = T;
-  lp.rot.freq_hi = L.freq_hi, lp.rot.freq_lo = L.freq_lo, lp.rot.pairs = L.rot_pairs, lp.rot.mag = L.rot_mag;
+  lp.rot.freq_hi = L.freq_hi, lp.rot.freq_lo = L.freq_lo, lp.rot.pairs = L.rot_pairs, lp.rot.mag = L.rot_mag, lp.rot.half = L.rot_layout == 0 ? 1 : 0;
   vra_stack_latent_prep(lp, dt_, stream);
   StkGemmArgs uq;
   uq.a = act_, uq.lda = L.q_rank, uq.w = L.uq, uq.M = T, uq.N = H * qd, uq.K = L.q_rank, uq.out = qkv_, uq.ldo = H * qd;
@@ -1093,7 +1105,8 @@ bool StackModel::mixer_latent(const StackLayer& L, const InputMetadata& md, int6
   a.positions = md.positions, a.block_tables = md.block_tables, a.context_lens = md.context_lens;
   a.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr;
   a.B = B, a.T = T, a.max_q = md.is_prefill ? md.max_seqlen_q : 1, a.H = H, a.G = 1, a.dim = kd, a.vdim = L.kv_rank;
-  a.BS = ec_.block_size, a.max_blocks = md.max_blocks, a.scale = L.scale;
+  a.BS = ec_.block_size, a.max_blocks = md.max_blocks, a.scale = L.scale, a.window = L.window;
+  if (L.head_gate) a.gate = z_ + L.q_rank + kd, a.gate_ld = L.nqkv();  // (a factor per row and head: it passes through W_uv)
   vra_stack_attention(a, dt_, stream);
   StkGemmArgs uv;  // per head: [T, kv_rank] x W_uv_h^T -> [T, vdim]
   uv.a = attn_, uv.lda = H * L.kv_rank, uv.a_batch_stride = L.kv_rank, uv.w = L.uv, uv.w_batch_stride = (int64_t)L.vdim * L.kv_rank, uv.batch = H;
@@ -1194,7 +1207,11 @@ bool StackModel::forward(const InputMetadata& md, int64_t stream, uint32_t* toke
   } else if (rows > logit_rows_cap_) {
     return error = "forward: more logit rows than the logits buffer holds", false;
   }
-  if (norm_kind_ == 1) {
+  if (norm_kind_ == 2) {  // (the seam's kernel without a sub-block's output: a norm of the row as it is)
+    StkSandwichArgs fn;
+    fn.x = const_cast<float*>(xin), fn.pre_w = final_norm_, fn.h = hl_, fn.T = rows, fn.W = W, fn.eps = eps_, fn.norm_kind = 2;
+    vra_stack_sandwich_norm(fn, dt_, stream);
+  } else if (norm_kind_ == 1) {
     // (the gathered rows are a copy: the kernel may read them through a non-const pointer, it adds nothing)
     vra_stack_dyt(const_cast<float*>(xin), nullptr, final_norm_, final_b_, final_alpha_, hl_, rows, W, dt_, stream);
   } else {
@@ -1203,7 +1220,7 @@ bool StackModel::forward(const InputMetadata& md, int64_t stream, uint32_t* toke
     vra_stack_group_norm(fn, dt_, stream);
   }
   StkGemmArgs hd;
-  hd.a = hl_, hd.lda = W, hd.w = head_, hd.M = rows, hd.N = vocab_, hd.K = W, hd.out = logits_, hd.ldo = vocab_, hd.out_f32 = 1, hd.alpha = logit_scale_;
+  hd.a = hl_, hd.lda = W, hd.w = head_, hd.M = rows, hd.N = vocab_, hd.K = W, hd.out = logits_, hd.ldo = vocab_, hd.out_f32 = 1, hd.alpha = logit_scale_, hd.softcap = logit_softcap_;
   vra_stack_gemm(hd, dt_, stream);
   if (tokens) vra_argmax_f32(logits_, tokens, rows, vocab_, stream);
   return !take_stack_err(error, "head");
@@ -1346,7 +1363,7 @@ bool StackModel::mixer_parallel(const StackLayer& L, const InputMetadata& md, in
 bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
   const int T = md.n_tokens, W = width_;
   hipStream_t st = reinterpret_cast<hipStream_t>(stream);
-  if (!md.state_slots || !md.prev_tokens) return error = "forward: this model needs the sequences' state slots and previous tokens", false;
+  if ((state_bytes_per_slot() > 0 && !md.state_slots) || (pair_buckets_ > 0 && !md.prev_tokens)) return error = "forward: this model needs the sequences' state slots and previous tokens", false;
   StkEmbedPairArgs e;
   e.ids = md.input_ids, e.positions = md.positions, e.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr, e.prev_tokens = md.prev_tokens;
   e.embed = embed_, e.table = pair_table_, e.buckets = pair_buckets_, e.mul_prev = pair_mul_prev_, e.mul_cur = pair_mul_cur_, e.scale = embed_scale_;
@@ -1356,12 +1373,12 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
   StkSandwichArgs pend;  // the parts of the last sub-block's output, not yet normed and added (post_w null: none)
   auto seam = [&](const float* pre_w, const float* pre_b, float pre_alpha, const StackLayer* router) {
     StkSandwichArgs s = pend;
-    s.x = x_, s.pre_w = pre_w, s.pre_b = pre_b, s.pre_alpha = pre_alpha, s.dyt = norm_kind_ == 1, s.h = h_, s.eps = eps_, s.T = T, s.W = W;
+    s.x = x_, s.pre_w = pre_w, s.pre_b = pre_b, s.pre_alpha = pre_alpha, s.norm_kind = norm_kind_, s.h = h_, s.eps = eps_, s.T = T, s.W = W;
     if (router) {
       s.router_w = router->router, s.router_bias = router->router_bias, s.n_router = router->experts + router->n_identity, s.top = router->top;
       s.pair_expert = pair_expert_, s.pair_weight = pair_weight_;
-      if (router->router_kind == 2) {
-        s.router_kind = 1, s.n_groups = router->n_groups, s.keep = router->keep, s.n_identity = router->n_identity;
+      if (router->router_kind >= 2) {
+        s.router_kind = router->router_kind - 1, s.n_groups = router->n_groups, s.keep = router->keep, s.n_identity = router->n_identity;
         if (router->n_identity > 0) s.h32 = h32_, s.id_weight = id_weight_;
       }
     }
@@ -1374,6 +1391,7 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
     if (!seam(L.norm_w, L.norm_b, L.norm_alpha, nullptr)) return false;
     bool ok = false;
     switch (L.mixer) {
+      case 1: ok = mixer_latent(L, md, stream); break;
       case 3: ok = mixer_delta(L, md, stream); break;
       case 4: ok = mixer_retention(L, md, stream); break;
       case 6: ok = mixer_lightning(L, md, stream); break;
@@ -1394,13 +1412,16 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
       vra_stack_moe_sort(pair_expert_, pair_weight_, P, L.top, L.experts, granule, rows, row_token_, row_scale_, row_pair_, tile_group_, stream);
       if (take_stack_err(error, "expert rows")) return false;
       // (the weights of a softmax router multiply the experts' OUTPUTS: the rows go in unscaled, the sum over a token's pairs carries them)
-      if (!expert_pair(h_, W, L.e_gu, (int64_t)2 * L.ffp * W, L.e_down, (int64_t)W * L.ffp, rows, L.ffp, L.ff, L.limit, tile_group_, granule, row_token_,
+      if (!expert_pair(h_, W, L.e_gu, (int64_t)(L.gated() ? 2 : 1) * L.ffp * W, L.e_down, (int64_t)W * L.ffp, rows, L.ffp, L.ff, L.limit, tile_group_, granule, row_token_,
                        L.router_kind >= 1 ? nullptr : row_scale_, row_pair_, pair_out_, stream, L.act_kind))
         return false;
       pend.p1 = pair_out_, pend.n1 = L.top, pend.pw = L.router_kind >= 1 ? pair_weight_ : nullptr;
       pend.post_w = L.post2_w, pend.post_b = L.post2_b, pend.post_alpha = L.post2_alpha;
       if (L.router_kind == 2 && L.n_identity > 0) {  // an identity expert's pair has no row: its weight times the feed-forward's own input
         pend.pe = pair_expert_, pend.p2 = h32_, pend.p2w = id_weight_, pend.c2 = 1.f;
+      } else if (L.shared_ff > 0) {  // the shared expert runs for every token and is added as it is
+        if (!expert_pair(h_, W, L.s_gu, 0, L.s_down, 0, T, L.sffp, L.shared_ff, L.shared_limit, nullptr, 0, nullptr, nullptr, nullptr, sh_, stream, L.act_kind)) return false;
+        pend.p2 = sh_, pend.c2 = 1.f;
       }
     } else if (L.mlp == 4) {
       if (!seam(L.norm2_w, L.norm2_b, L.norm2_alpha, nullptr)) return false;

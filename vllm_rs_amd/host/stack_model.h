@@ -4,15 +4,18 @@
 //   block   parallel:    x <- x + m * (mixer(h) + ff(h)),  h = norm(x)                      (Ditilix)
 //           sequential:  x <- x + mixer(norm1(x)),  x <- x + ff(norm2(x))                   (Gaperax)
 //           sandwich:    x <- x + norm1b(mixer(norm1(x))),  x <- x + norm2b(ff(norm2(x)))   (Zifetar: RMS norms, norm_offset added to the weights;
-//                        Sudosun: Dynamic Tanh norms, the head is the embedding table)
-//   norm    rms: RMS norm over `groups` equal parts of the width;  dyt: Dynamic Tanh  tanh(alpha x) w + b  (no statistics)
+//                        Sudosun: Dynamic Tanh norms, the head is the embedding table;
+//                        Pesivik: layer norms, layer_scale: each sub-block's normed output times one factor per channel)
+//   norm    rms: RMS norm over `groups` equal parts of the width;  dyt: Dynamic Tanh  tanh(alpha x) w + b  (no statistics);
+//           layer: (x - mean) / sqrt(variance + eps) w  (sandwich blocks)
 //   pos     sinusoid: a position vector added to the embedding;  none: positions enter inside the mixers
 //   embedding (sandwich stacks): embed * embed_scale + a row of a hashed (previous token, token) table (pair_buckets, pair_mul_prev,
 //           pair_mul_cur; the table's last row for a sequence's first token), then an RMS norm of its own
 //   mixer   attention: causal softmax, query temperature, soft cap, grouped key/value heads, optionally another layer's keys / values
 //           latent:    queries and keys / values through low-rank latents, a rotated key part shared by the heads (rotary with optional
 //                      YaRN scaling), a softmax sink per head; the cache holds one row [latent | rotated part] per token and the
-//                      up-projections are absorbed: q' = [W_uk_h^T q_h | rot(q_h)], values = the latent, W_uv_h after the sum over keys
+//                      up-projections are absorbed: q' = [W_uk_h^T q_h | rot(q_h)], values = the latent, W_uv_h after the sum over keys;
+//                      optionally a sliding window, a sigmoid output gate per head, rotary in the rotate-half layout
 //           sigmoid:   biased q / k / v, one RMS norm over all of q and all of k, weights sigmoid(score - slope_h * distance + bias_h)
 //                      without normalisation, a window that keeps the first tokens, heads mixed by a matrix, a sigmoid output gate
 //   delta:     gated delta rule: short causal convolutions + silu on q / k / v, unit-vector q and k, a write strength per head, a decay per
@@ -32,7 +35,11 @@
 //   mlp     none | dense (PolyNorm activation) | moe (sigmoid router, clamped gated experts, gated shared expert) | gated (gelu_tanh(gate) * up)
 //           | clamped (dense, the clamped gated form of the experts above);  moe with router=softmax_all: scores are a softmax over all
 //           router outputs, a correction is added for the choice only, the choice is restricted to the best `keep` of `groups` groups of
-//           neighbouring experts, the weights are the plain scores, and the last `identity` outputs are experts that return their input
+//           neighbouring experts, the weights are the plain scores, and the last `identity` outputs are experts that return their input;
+//           moe with router=sigmoid_norm: sigmoid scores, the correction and the groups as before (a group's worth is the sum of its two best
+//           corrected scores), weights = the chosen scores divided by their sum; a shared expert may run beside it, added as it is;
+//           act=gelu: experts (and the shared one) without a gate, down(gelu(up h)) with the exact (erf) gelu
+//   logit_softcap: logits <- cap * tanh(logits / cap)
 //   sandwich blocks with norm=dyt use Dynamic Tanh for all four norms of a layer; tie_head=1: the head is the embedding table
 //   weights_of=j: the layer runs with layer j's tensors and a cache of its own
 // vllm_rs_amd/checkpoint.py turns a design's config.json into the spec text below.
@@ -41,15 +48,16 @@
 // activations are bf16 (f32 accumulation) or, for a VRA_F32 model, f32 throughout.
 //
 // Spec text, one record per line, `key=value` fields:
-//   stack width=.. vocab=.. eps=.. groups=.. residual_mult=.. logit_scale=.. pos_base=.. block=.. norm=.. pos=..
+//   stack width=.. vocab=.. eps=.. groups=.. residual_mult=.. logit_scale=.. logit_softcap=.. pos_base=.. block=.. norm=.. pos=.. layer_scale=0|1
 //   layer mixer=.. heads=.. kv_heads=.. dim=.. vdim=.. scale=.. softcap=.. temp_coef=.. temp_every=.. kv_from=.. weights_of=..
 //         rot_dim=.. kv_rank=.. q_rank=.. rot_dims=.. rot_base=.. yarn_factor=.. yarn_original=.. yarn_fast=.. yarn_slow=.. sink=0|1
 //         window=.. keep_first=.. slope_exp=..
 //         conv=.. rank_a=.. rank_g=.. decay=d0,d1,.. chunk=.. qk_norm=0|1 bias=0|1 rs_factor=.. rs_low=.. rs_high=.. rs_original=..
 //         r_heads=.. r_dim=.. r_vdim=.. tau=.. left_scale=.. right_scale=..
-//         lowrank=0|1 right=gla|rglru r_width=.. r_blocks=.. r_conv=.. head_temp=0|1 head_gate=0|1 rot_layout=half|pairs branch_norm=0|1
-//         mlp=none|dense|moe|gated|clamped ff=.. experts=.. top=.. limit=.. shared_ff=.. shared_limit=.. router=sigmoid|softmax|softmax_all
-//         act=clamped|silu identity=.. groups=.. keep=..
+//         lowrank=0|1 right=gla|rglru r_width=.. r_blocks=.. r_conv=.. head_temp=0|1 head_gate=0|1 branch_norm=0|1
+//         rot_layout=half|pairs (latent: pairs unless given, the other mixers: half)
+//         mlp=none|dense|moe|gated|clamped ff=.. experts=.. top=.. limit=.. shared_ff=.. shared_limit=.. router=sigmoid|softmax|softmax_all|sigmoid_norm
+//         act=clamped|silu|gelu identity=.. groups=.. keep=..
 #pragma once
 #include <map>
 #include <string>
@@ -83,14 +91,16 @@ struct StackLayer {
   // of r_width channels with r_blocks gate blocks behind a convolution of `conv` taps; the left branch's per-head temperature and output
   // gate, rotary layout (1 = neighbouring pairs), a norm per branch before the sum
   int lowrank = 1, right_kind = 0, r_width = 0, r_blocks = 1, head_temp = 0, head_gate = 0, rot_layout = 0, branch_norm = 0;
-  // router_kind 2: identity experts and expert groups
+  // router_kind 2 / 3: identity experts (2) and expert groups
   int n_identity = 0, n_groups = 0, keep = 0;
   // feed-forward: 0 none, 1 dense (PolyNorm), 2 mixture of experts, 3 gated dense (gelu_tanh(gate) * up), 4 clamped gated dense
   int mlp = 0, ff = 0, experts = 0, top = 0, shared_ff = 0;
   float limit = 0.f, shared_limit = 0.f;
   // mixture of experts: router 0 = sigmoid scores as weights on the experts' inputs, 1 = biased logits, softmax over the chosen ones, weights
-  // on the experts' outputs; act 0 = clamped gated form, 2 = silu(gate) * up
+  // on the experts' outputs, 2 = softmax over all outputs with corrected choice, 3 = normalised sigmoid scores with corrected choice;
+  // act 0 = clamped gated form, 2 = silu(gate) * up, 3 = exact gelu of up, no gate
   int router_kind = 0, act_kind = 0;
+  bool gated() const { return act_kind != 3; }
   // derived
   int cache = -1;          // index of the paged cache this layer reads (its own, or the one of layer kv_from)
   bool owns_cache = false;
@@ -98,9 +108,9 @@ struct StackLayer {
   int nq() const { return heads * (mixer == 1 ? dim + rot_dim : dim); }
   int nk() const { return kv_heads * dim; }
   int nv() const { return kv_heads * vdim; }
-  // columns of the joint input projection: q (| k | v) of softmax attention, q | k | v | gate of sigmoid attention, the three latents
+  // columns of the joint input projection: q (| k | v) of softmax attention, q | k | v | gate of sigmoid attention, the three latents (| head gates)
   int nqkv() const {
-    if (mixer == 1) return q_rank + kv_rank + rot_dim;
+    if (mixer == 1) return q_rank + kv_rank + rot_dim + (head_gate ? heads : 0);
     if (mixer == 2) return nq() + nk() + nv() + heads * vdim;
     if (mixer == 3) return 2 * nk() + heads * vdim + heads + (lowrank ? 0 : heads + heads * vdim);  // q | k (kv_heads each) | v | write strengths (| decays | gate)
     if (mixer == 4 || mixer == 6) return 2 * heads * dim + 2 * heads * vdim;       // q | k | v | gate
@@ -137,7 +147,7 @@ struct StackLayer {
   void* down = nullptr;    // dense [width, ff]
   float* act = nullptr;    // PolyNorm a, b, c, e
   void* router = nullptr;  // [experts (+ 1: the shared expert's gate), width]
-  void* e_gu = nullptr;    // [experts][2 * ffp][width], gate / up rows interleaved in blocks of 16
+  void* e_gu = nullptr;    // [experts][2 * ffp][width], gate / up rows interleaved in blocks of 16 (experts without a gate: [experts][ffp][width])
   void* e_down = nullptr;  // [experts][width][ffp]
   void* s_gu = nullptr;    // [2 * sffp][width]  (shared expert, or the gated dense feed-forward)
   void* s_down = nullptr;  // [width][sffp]
@@ -220,9 +230,10 @@ class StackModel : public ModelBase {
   int dt_ = 0;
   size_t es_ = 2;
   int width_ = 0, vocab_ = 0, groups_ = 1;
-  int block_ = 0, norm_kind_ = 0, pos_kind_ = 0;  // 0 parallel / rms / sinusoid, 1 sequential / dyt / none, block 2 sandwich
+  int block_ = 0, norm_kind_ = 0, pos_kind_ = 0;  // 0 parallel / rms / sinusoid, 1 sequential / dyt / none, block 2 sandwich, norm 2 layer norm
   float norm_offset_ = 0.f, embed_scale_ = 1.f;    // added to every norm weight at load; multiplies the embedding row
-  int embed_norm_ = 0, pair_buckets_ = 0, tie_head_ = 0;
+  int embed_norm_ = 0, pair_buckets_ = 0, tie_head_ = 0, layer_scale_ = 0;
+  float logit_softcap_ = 0.f;
   float *h32_ = nullptr, *id_weight_ = nullptr;  // identity experts: the unrounded feed-forward input and the summed weight of a token's identity picks
   int64_t pair_mul_prev_ = 0, pair_mul_cur_ = 0;
   void* pair_table_ = nullptr;
