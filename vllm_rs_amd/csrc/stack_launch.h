@@ -115,6 +115,9 @@ struct StkAttnArgs {
   int gate_ld = 0;
 };
 void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream);
+// its shared-row form on the matrix cores (stack_latent.hip): bf16 prompt steps with G = 1 and vc = kc, rows up to 576 wide, values up to 512;
+// false: not a shape of that kernel, nothing was launched
+bool vra_stack_latent_prefill(const StkAttnArgs& a, int dtype, int64_t stream);
 
 // rows of a [*, W] f32 matrix picked by index -> dst (f32)
 void vra_stack_gather_rows_f32(const float* src, const uint32_t* rows, float* dst, int n, int W, int64_t stream);

@@ -1102,6 +1102,7 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
 #undef STK_DEC
     return;
   }
+  if (vra_stack_latent_prefill(a, dtype, stream)) return;
   if (dtype == VRA_BF16 && a.dim % 8 == 0 && a.vdim % 16 == 0 && a.dim <= 256 && a.vdim <= 256 && a.ldq % 8 == 0 && ((uintptr_t)a.q % 16 == 0) && a.BS % 32 == 0 &&
       a.k_ld % 8 == 0 && a.v_ld % 8 == 0 && ((uintptr_t)a.vc % 16 == 0)) {
     dim3 grid((a.max_q + 63) / 64, a.B, a.H);

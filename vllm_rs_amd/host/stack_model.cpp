@@ -172,7 +172,7 @@ bool StackModel::parse_spec(const char* spec) {
       L.weights_of = root;
       const StackLayer& S = layers_[root];
       if (S.mixer != L.mixer || S.heads != L.heads || S.kv_heads != L.kv_heads || S.dim != L.dim || S.vdim != L.vdim || S.rot_dim != L.rot_dim ||
-          S.kv_rank != L.kv_rank || S.q_rank != L.q_rank || S.window != L.window || S.head_gate != L.head_gate || S.experts != L.experts || S.shared_ff != L.shared_ff || S.mlp != L.mlp || S.ff != L.ff || S.kv_from >= 0 || L.kv_from >= 0)
+          S.kv_rank != L.kv_rank || S.q_rank != L.q_rank || S.window != L.window || S.head_gate != L.head_gate || (L.mlp == 2 && (S.experts != L.experts || S.shared_ff != L.shared_ff)) || S.mlp != L.mlp || S.ff != L.ff || S.kv_from >= 0 || L.kv_from >= 0)
         return spec_error_ = "layer stack spec: a layer that shares weights has the shapes of the layer it names" + at, false;
     }
     if (!L.has_cache()) {
