@@ -113,10 +113,18 @@ struct StkAttnArgs {
   const float* head_scale = nullptr;  // f32 [H]: head h's scores are also multiplied by head_scale[h] (the sink is not)
   const float* gate = nullptr;  // f32 [T, gate_ld], column h: head h's output row is multiplied by sigmoid(gate[t, h])
   int gate_ld = 0;
+  // latent decode form: f32 scratch of B * splits * H * (vdim + 2) floats for the parts of the key range (null: the one-launch kernel)
+  float* scratch = nullptr;
+  size_t scratch_bytes = 0;
+  int splits = 0;
 };
 void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream);
 // its shared-row form on the matrix cores (stack_latent.hip): bf16 prompt steps with G = 1 and vc = kc, rows up to 576 wide, values up to 512;
 // false: not a shape of that kernel, nothing was launched
+// vra_stack_latent_decode: the same for one token per sequence, in two launches over `splits` parts of the key range (any number from 1 to 64; it
+// fixes the order of the sums: vra_stack_latent_splits names one for a model)
+int vra_stack_latent_splits(int window, int max_len, int max_seqs, int heads, int vdim);
+bool vra_stack_latent_decode(const StkAttnArgs& a, int dtype, int64_t stream);
 bool vra_stack_latent_prefill(const StkAttnArgs& a, int dtype, int64_t stream);
 
 // rows of a [*, W] f32 matrix picked by index -> dst (f32)

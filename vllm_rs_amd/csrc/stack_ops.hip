@@ -1088,6 +1088,7 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
                 "stack attention: heads must be a multiple of kv heads, value size at most 512");
   hipStream_t st = as_stream(stream);
   if (!a.cu_q) {
+    if (vra_stack_latent_decode(a, dtype, stream)) return;
     const size_t lds = ((size_t)a.dim + 2 * STK_DW * 64 + 2 * STK_DW + STK_DW * (size_t)a.vdim) * sizeof(float);
     VRA_CHECK_ARG(lds <= 64 * 1024, "stack attention: head does not fit LDS");
     dim3 grid(a.B, a.H);

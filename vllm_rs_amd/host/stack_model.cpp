@@ -955,6 +955,12 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
     sig_scratch_bytes_ = std::max(sig_scratch_bytes_, (size_t)max_seqs * 64 * hv * 4);
   }
   if (sig_scratch_bytes_ && !(sig_scratch_ = (float*)dalloc(sig_scratch_bytes_))) return false;
+  for (const StackLayer& L : layers_) {
+    if (L.mixer != 1 || dt_ != VRA_BF16) continue;
+    const int s = vra_stack_latent_splits(L.window, mc_.max_position_embeddings, max_seqs, L.heads, L.kv_rank);
+    lat_scratch_bytes_ = std::max(lat_scratch_bytes_, (size_t)max_seqs * s * L.heads * (L.kv_rank + 2) * 4);
+  }
+  if (lat_scratch_bytes_ && !(lat_scratch_ = (float*)dalloc(lat_scratch_bytes_))) return false;
   if (want_h32 && (!(h32_ = (float*)dalloc(T * W * 4)) || !(id_weight_ = (float*)dalloc(T * 4)))) return false;
   const size_t P = T * std::max<size_t>(top, 1);
   if (!(pair_expert_ = (int*)dalloc(P * 4)) || !(pair_weight_ = (float*)dalloc(P * 4)) || !(gate_ = (float*)dalloc(T * 4)) ||
@@ -1106,6 +1112,7 @@ bool StackModel::mixer_latent(const StackLayer& L, const InputMetadata& md, int6
   a.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr;
   a.B = B, a.T = T, a.max_q = md.is_prefill ? md.max_seqlen_q : 1, a.H = H, a.G = 1, a.dim = kd, a.vdim = L.kv_rank;
   a.BS = ec_.block_size, a.max_blocks = md.max_blocks, a.scale = L.scale, a.window = L.window;
+  a.scratch = lat_scratch_, a.scratch_bytes = lat_scratch_bytes_, a.splits = vra_stack_latent_splits(L.window, mc_.max_position_embeddings, max_seqs_, H, L.kv_rank);
   if (L.head_gate) a.gate = z_ + L.q_rank + kd, a.gate_ld = L.nqkv();  // (a factor per row and head: it passes through W_uv)
   vra_stack_attention(a, dt_, stream);
   StkGemmArgs uv;  // per head: [T, kv_rank] x W_uv_h^T -> [T, vdim]

@@ -1,5 +1,6 @@
-"""Throughput of a layer-stack model (Ditilix, Gaperax, Zifetar or Sudosun design) beside the dense bf16 Llama of the same widths —
-`python bench.py --design ditilix|gaperax|zifetar|sudosun` (Sudosun also beside the Zifetar design of the same widths, its closest model;
+"""Throughput of a layer-stack model (Ditilix, Gaperax, Zifetar, Sudosun or Pesivik design) beside the dense bf16 Llama of the same widths —
+`python bench.py --design ditilix|gaperax|zifetar|sudosun|pesivik` (Pesivik also beside a Gaperax stack whose layers are all latent attention
+with the same latents, and beside the Sudosun design of the same widths and experts; Sudosun also beside the Zifetar design of the same widths, its closest model;
 Zifetar also beside the Ditilix mixture of experts of the same widths, the closest
 model of its class).
 
@@ -151,6 +152,35 @@ def sudosun_costs(cj):
     return 2 * n, 2 * n
 
 
+def pesivik_config(width, heads, dim, layers, vocab, kv_rank, q_rank, rot_dim, window, experts, top, expert_ff, shared_ff, groups, keep):
+    """config.json dict of a Pesivik model: every layer latent attention under a window and a mixture of experts with a shared one"""
+    mx = dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=dim, kv_rank=kv_rank, q_rank=q_rank, scale=(dim + rot_dim) ** -0.5, mask=dict(size=window),
+              rot=dict(base=1e6, dims=rot_dim))
+    mlp = dict(kind="moe", expert=dict(ff=expert_ff), router=dict(experts=experts, top=top, groups=dict(count=groups, keep=keep)), shared=dict(ff=shared_ff))
+    return dict(architecture="Pesivik", width=width, vocab=vocab, norm=dict(eps=1e-5), embedding=dict(scale=width ** 0.5), logit_softcap=50.0,
+                layers=[dict(type="latent_attention", mixer=mx, mlp=mlp) for _ in range(layers)])
+
+
+def pesivik_costs(cj):
+    """(matrix FLOPs per token without attention, weight bytes a one-token step reads) of a Pesivik config"""
+    W, n = cj["width"], 0
+    for layer in cj["layers"]:
+        mx, mlp = layer["mixer"], layer.get("mlp")
+        H, dim, vdim, rd, kr, qr = (mx[k] for k in ("heads", "dim", "vdim", "rot_dim", "kv_rank", "q_rank"))
+        n += W * (qr + kr + rd + H) + qr * H * (dim + rd) + H * dim * kr + H * kr * vdim + H * vdim * W
+        if mlp:
+            n += mlp["router"]["top"] * 2 * W * mlp["expert"]["ff"] + W * mlp["router"]["experts"] + (2 * W * mlp["shared"]["ff"] if mlp.get("shared") else 0)
+    n += cj["vocab"] * W
+    return 2 * n, 2 * n
+
+
+def latent_gaperax_config(width, heads, dim, ff, layers, vocab, kv_rank, q_rank, rot_dim):
+    """a Gaperax stack whose layers are all latent attention"""
+    cj = gaperax_config(width, heads, heads, dim, ff, layers, vocab, kv_rank, q_rank, rot_dim, 0, 0)
+    cj["layers"] = [dict(cj["layers"][0]) for _ in range(layers)]
+    return cj
+
+
 def llama_costs(cfg):
     H, D = cfg["hidden_size"], cfg["head_dim"]
     per = H * (cfg["num_heads"] + 2 * cfg["num_kv_heads"]) * D + cfg["num_heads"] * D * H + 3 * H * cfg["intermediate_size"]
@@ -221,14 +251,26 @@ SUDOSUN_SIZES = {
 }
 
 
+PESIVIK_SIZES = {
+    # name: (width, heads, head size, layers, vocab, kv latent, q latent, rotated part, window, experts, top, expert ff, shared ff, groups, kept)
+    "pesivik-2048": (2048, 16, 128, 3, 32000, 192, 768, 64, 1024, 16, 2, 1024, 2048, 4, 2),
+    "pesivik-2048-kv512": (2048, 16, 128, 3, 32000, 512, 1536, 64, 1024, 32, 4, 1024, 2048, 8, 4),
+    "pesivik-4096-kv512": (4096, 32, 128, 3, 32000, 512, 1536, 64, 1024, 16, 2, 2048, 2048, 4, 2),
+}
+
+
 def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design="ditilix"):
     from . import _lib, checkpoint
     from .engine import BF16, Engine
     L = _lib.load()
     lines = []
-    table = GAPERAX_SIZES if design == "gaperax" else (ZIFETAR_SIZES if design == "zifetar" else (SUDOSUN_SIZES if design == "sudosun" else SIZES))
+    table = GAPERAX_SIZES if design == "gaperax" else (ZIFETAR_SIZES if design == "zifetar" else (SUDOSUN_SIZES if design == "sudosun" else (PESIVIK_SIZES if design == "pesivik" else SIZES)))
     for name in (sizes or table):
-        if design == "sudosun":
+        if design == "pesivik":
+            width, heads, dim, layers, vocab, kr, qr, rd, window, experts, top, eff, sff, groups, keep = table[name]
+            cj = pesivik_config(width, heads, dim, layers, vocab, kr, qr, rd, window, experts, top, eff, sff, groups, keep)
+            kvh, ff = heads // 4, 4 * width
+        elif design == "sudosun":
             width, heads, kvh, dim, layers, vocab, experts, top, eff, window, blocks = table[name]
             cj = sudosun_config(width, heads, kvh, dim, layers, vocab, experts, top, eff, window, blocks)
             ff = 4 * width
@@ -246,7 +288,16 @@ def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design
         res = dict(stack=measure(eng, L, vocab, prefill_tokens, steps, warmup))
         eng.close()
         res["stack"]["flops_per_token"], res["stack"]["weight_bytes_per_step"] = (
-            sudosun_costs(cj) if design == "sudosun" else (zifetar_costs(cj) if design == "zifetar" else (gaperax_costs(cj) if design == "gaperax" else stack_costs(cj))))
+            pesivik_costs(cj) if design == "pesivik" else (sudosun_costs(cj) if design == "sudosun" else (zifetar_costs(cj) if design == "zifetar" else (gaperax_costs(cj) if design == "gaperax" else stack_costs(cj)))))
+        if design == "pesivik":  # the two closest models: latent attention with the same latents (dense gated feed-forward); the sandwich seams
+            # and mixture of experts of the Sudosun design (recurrent mixers)
+            gj = latent_gaperax_config(width, heads, dim, ff, layers, vocab, kr, qr, rd)
+            sj = sudosun_config(width, heads, kvh, dim, layers, vocab, experts, top, eff, window, heads)
+            for key, other, costs in (("gaperax_latent", gj, gaperax_costs), ("sudosun", sj, sudosun_costs)):
+                eng = Engine(checkpoint.parse_config(other), num_gpu_blocks=512, max_num_seqs=8, max_model_len=4096, use_graph=graph).init_synthetic()
+                res[key] = measure(eng, L, vocab, prefill_tokens, steps, warmup)
+                eng.close()
+                res[key]["flops_per_token"], res[key]["weight_bytes_per_step"] = costs(other)
         if design == "sudosun":  # the closest model of the same class: the Zifetar design of the same widths (state mixers, the same experts)
             zj = zifetar_config(width, heads, kvh, dim, layers, vocab, experts, top, eff, window, width // 32)
             eng = Engine(checkpoint.parse_config(zj), num_gpu_blocks=512, max_num_seqs=8, max_model_len=4096, use_graph=graph).init_synthetic()
@@ -269,7 +320,7 @@ def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design
         for m in res.values():
             m["prefill_matrix_tflops"] = m["prefill_tokens_per_s"] * m["flops_per_token"] / 1e12
             m["decode_bs1_weight_gb_per_s"] = m["weight_bytes_per_step"] / (m["decode_bs1_ms_per_step"] / 1e3) / 1e9
-        line = dict(metric="stack_vs_dense_llama", size=name, design={"gaperax": "Gaperax", "zifetar": "Zifetar", "sudosun": "Sudosun"}.get(design, "Ditilix"), dtype="bf16", data="synthetic", prefill_tokens=prefill_tokens,
+        line = dict(metric="stack_vs_dense_llama", size=name, design={"gaperax": "Gaperax", "zifetar": "Zifetar", "sudosun": "Sudosun", "pesivik": "Pesivik"}.get(design, "Ditilix"), dtype="bf16", data="synthetic", prefill_tokens=prefill_tokens,
                     decode_context=512, steps=steps, **res)
         print(json.dumps(line), flush=True)
         lines.append(line)
