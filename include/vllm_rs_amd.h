@@ -662,10 +662,10 @@ void vra_stack_op_dyt(float* x, const float* add, const float* w, const float* b
 void vra_stack_op_latent_prep(const float* raw, int32_t ld, int32_t q_rank, int32_t kv_rank, int32_t rot_dim, const float* qn_w,
                               const float* kvn_w, float eps, void* cq, void* cache, int32_t cache_ld, const int64_t* slots,
                               const int64_t* positions, const float* freq_hi, const float* freq_lo, int32_t pairs, float mag,
-                              int32_t T, int32_t dtype, int64_t stream);
+                              int32_t half, int32_t T, int32_t dtype, int64_t stream);
 void vra_stack_op_rope_heads(const void* in, int32_t in_ld, int32_t in_hs, int32_t in_off, void* out, int32_t out_ld, int32_t out_hs,
                              int32_t out_off, int32_t n, int32_t H, const int64_t* positions, const float* freq_hi,
-                             const float* freq_lo, int32_t pairs, float mag, int32_t T, int32_t dtype, int64_t stream);
+                             const float* freq_lo, int32_t pairs, float mag, int32_t half, int32_t T, int32_t dtype, int64_t stream);
 void vra_stack_op_qk_norm_store(const float* raw, int32_t ld, int32_t nq, int32_t nk, int32_t nv, const float* q_w, const float* k_w,
                                 float eps, void* q_out, void* kc, void* vc, const int64_t* slots, int32_t T, int32_t dtype,
                                 int64_t stream);
@@ -733,6 +733,21 @@ void vra_stack_op_linear_scan_ex(const float* q, int32_t ldq, const float* k, in
                                  int32_t ldb, float q_scale, float* state, const int32_t* state_slots, const int64_t* positions,
                                  const uint32_t* cu_q, float* out, int32_t ldo, int32_t B, int32_t H, int32_t qk_rep, int32_t dim,
                                  int32_t vdim, int64_t stream);
+
+/* attention_latent: the softmax attention over a latent cache (csrc/stack_latent.hip): one row of k_ld elements per token, keys = its first
+ * `dim` columns for every head, values = its first vdim columns; window, sink, head_scale, gate as in attention_window.  Decode form
+ * (cu_q null) with scratch: B * splits * H * (vdim + 2) floats, the key range in `splits` parts.
+ * gemm_post: vra_stack_op_gemm with bias and the element-wise epilogues: epi 2 = act(alpha sum + bias) (act 3: exact gelu),
+ * softcap > 0: softcap tanh(v / softcap). */
+void vra_stack_op_attention_latent(const void* q, int32_t ldq, void* out, const void* cache, int32_t k_ld, const int64_t* positions,
+                                   const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_q, int32_t B, int32_t T,
+                                   int32_t max_q, int32_t H, int32_t dim, int32_t vdim, int32_t BS, int32_t max_blocks, float scale,
+                                   int32_t window, const float* sink, const float* head_scale, const float* gate, int32_t gate_ld,
+                                   float* scratch, int64_t scratch_bytes, int32_t splits, int32_t dtype, int64_t stream);
+void vra_stack_op_gemm_post(const void* a, int32_t lda, const void* w, int64_t w_group_stride, void* out, int32_t ldo, int32_t out_f32,
+                            int32_t M, int32_t N, int32_t K, float alpha, const float* bias, const int32_t* tile_group, int32_t granule,
+                            const int32_t* a_row, const int32_t* out_row, int32_t epi, int32_t act, float softcap, int32_t dtype,
+                            int64_t stream);
 
 /* decode-step microbenchmark hook used by bench.py: runs `steps` decode steps of the current
  * running batch back to back (graph replay when enabled) and returns elapsed ms measured with HIP

@@ -152,7 +152,7 @@ def test_latent_rows_norms_rotary_cache(dt, rot):
     fh, fl, mag = freq_pair(rot)
     cq, cache = empty(T * qr * 4), empty(20 * (kr + rd) * 4)
     L.vra_stack_op_latent_prep(f32(raw_rows).ptr, qr + kr + rd, qr, kr, rd, f32(qn).ptr, f32(kn).ptr, 1e-5, cq.ptr, cache.ptr, kr + rd, raw(slots, np.int64).ptr,
-                               raw(pos, np.int64).ptr, f32(fh).ptr, f32(fl).ptr, rot["dims"] // 2, mag, T, dt, 0)
+                               raw(pos, np.int64).ptr, f32(fh).ptr, f32(fl).ptr, rot["dims"] // 2, mag, 0, T, dt, 0)
     check()
     x = raw_rows.astype(np.float64)
     tol = 2e-6 if dt == F32 else 4e-3
@@ -179,7 +179,7 @@ def test_rotary_on_head_rows(dt):
     out = empty(T * H * hs_out * 4).fill_bytes(0)
     fh, fl, mag = freq_pair(rot)
     L.vra_stack_op_rope_heads(to_dev(x.reshape(T, -1), dt).ptr, H * hs_in, hs_in, off_in, out.ptr, H * hs_out, hs_out, off_out, n, H, raw(pos, np.int64).ptr,
-                              f32(fh).ptr, f32(fl).ptr, rot["dims"] // 2, mag, T, dt, 0)
+                              f32(fh).ptr, f32(fl).ptr, rot["dims"] // 2, mag, 0, T, dt, 0)
     check()
     got = from_dev(out, (T, H, hs_out), dt)
     want = go.rotate_pairs(x[:, :, off_in:off_in + n].astype(np.float64), *go.rotary_table(rot, pos))

@@ -208,8 +208,8 @@ def load():
     _sig(lib, "vra_stack_op_attention", None, P, c_i32, P, P, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32,
          c_f32, c_f32, c_f32, c_i32, c_i32, c_i64)
     _sig(lib, "vra_stack_op_dyt", None, P, P, P, P, c_f32, P, c_i32, c_i32, c_i32, c_i64)
-    _sig(lib, "vra_stack_op_latent_prep", None, P, c_i32, c_i32, c_i32, c_i32, P, P, c_f32, P, P, c_i32, P, P, P, P, c_i32, c_f32, c_i32, c_i32, c_i64)
-    _sig(lib, "vra_stack_op_rope_heads", None, P, c_i32, c_i32, c_i32, P, c_i32, c_i32, c_i32, c_i32, c_i32, P, P, P, c_i32, c_f32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_latent_prep", None, P, c_i32, c_i32, c_i32, c_i32, P, P, c_f32, P, P, c_i32, P, P, P, P, c_i32, c_f32, c_i32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_rope_heads", None, P, c_i32, c_i32, c_i32, P, c_i32, c_i32, c_i32, c_i32, c_i32, P, P, P, c_i32, c_f32, c_i32, c_i32, c_i32, c_i64)
     _sig(lib, "vra_stack_op_qk_norm_store", None, P, c_i32, c_i32, c_i32, c_i32, P, P, c_f32, P, P, P, P, c_i32, c_i32, c_i64)
     _sig(lib, "vra_stack_op_sigmoid_attention", None, P, c_i32, P, P, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32,
          c_f32, c_i32, c_i32, P, P, P, P, c_i32, P, c_i64, c_i32, c_i32, c_i64)
@@ -229,6 +229,10 @@ def load():
     _sig(lib, "vra_stack_op_gated_scan", None, P, c_i32, P, P, c_i32, c_i32, P, c_i32, P, c_f32, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i64)
     _sig(lib, "vra_stack_op_linear_scan_ex", None, P, c_i32, P, c_i32, P, c_i32, P, c_i32, c_i32, c_i32, P, P, c_i32, c_f32, P, P, P, P, P, c_i32, c_i32,
          c_i32, c_i32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_attention_latent", None, P, c_i32, P, P, c_i32, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_f32, c_i32,
+         P, P, P, c_i32, P, c_i64, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_gemm_post", None, P, c_i32, P, c_i64, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_f32, P, P, c_i32, P, P, c_i32, c_i32, c_f32,
+         c_i32, c_i64)
     _sig(lib, "vra_engine_create_spec", P, MC, EC, C.c_char_p)
     _sig(lib, "vra_engine_replay_step", c_i32, P, c_i32, P, P, P, P, P, c_i32, P, P)
     _sig(lib, "vra_engine_debug_layer_trace", None, P, c_i32)

@@ -478,3 +478,18 @@ bool vra_stack_latent_prefill(const StkAttnArgs& a, int dtype, int64_t stream) {
 #undef STK_LAT
   return true;
 }
+
+// softmax attention over latent rows (keys: whole rows of k_ld elements, values: their first vdim columns) with window, sink, scale and output
+// gate per head; scratch (may be null) and splits: the decode form in parts
+extern "C" void vra_stack_op_attention_latent(const void* q, int32_t ldq, void* out, const void* cache, int32_t k_ld, const int64_t* positions,
+                                              const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_q, int32_t B, int32_t T,
+                                              int32_t max_q, int32_t H, int32_t dim, int32_t vdim, int32_t BS, int32_t max_blocks, float scale, int32_t window,
+                                              const float* sink, const float* head_scale, const float* gate, int32_t gate_ld, float* scratch,
+                                              int64_t scratch_bytes, int32_t splits, int32_t dtype, int64_t stream) {
+  StkAttnArgs a;
+  a.q = q, a.ldq = ldq, a.out = out, a.kc = cache, a.vc = cache, a.k_ld = k_ld, a.v_ld = k_ld, a.positions = positions, a.block_tables = block_tables;
+  a.context_lens = context_lens, a.cu_q = cu_q, a.B = B, a.T = T, a.max_q = max_q, a.H = H, a.G = 1, a.dim = dim, a.vdim = vdim, a.BS = BS;
+  a.max_blocks = max_blocks, a.scale = scale, a.window = window, a.sink = sink, a.head_scale = head_scale, a.gate = gate, a.gate_ld = gate_ld;
+  a.scratch = scratch, a.scratch_bytes = (size_t)scratch_bytes, a.splits = splits;
+  vra_stack_attention(a, dtype, stream);
+}

@@ -941,19 +941,19 @@ extern "C" void vra_stack_op_dyt(float* x, const float* add, const float* w, con
 }
 extern "C" void vra_stack_op_latent_prep(const float* raw, int32_t ld, int32_t q_rank, int32_t kv_rank, int32_t rot_dim, const float* qn_w,
                                          const float* kvn_w, float eps, void* cq, void* cache, int32_t cache_ld, const int64_t* slots,
-                                         const int64_t* positions, const float* freq_hi, const float* freq_lo, int32_t pairs, float mag, int32_t T,
-                                         int32_t dtype, int64_t stream) {
+                                         const int64_t* positions, const float* freq_hi, const float* freq_lo, int32_t pairs, float mag, int32_t half,
+                                         int32_t T, int32_t dtype, int64_t stream) {
   StkLatentPrepArgs a;
   a.raw = raw, a.ld = ld, a.q_rank = q_rank, a.kv_rank = kv_rank, a.rot_dim = rot_dim, a.qn_w = qn_w, a.kvn_w = kvn_w, a.eps = eps, a.cq = cq;
   a.cache = cache, a.cache_ld = cache_ld, a.slots = slots, a.positions = positions, a.T = T;
-  a.rot.freq_hi = freq_hi, a.rot.freq_lo = freq_lo, a.rot.pairs = pairs, a.rot.mag = mag;
+  a.rot.freq_hi = freq_hi, a.rot.freq_lo = freq_lo, a.rot.pairs = pairs, a.rot.mag = mag, a.rot.half = half;
   vra_stack_latent_prep(a, dtype, stream);
 }
 extern "C" void vra_stack_op_rope_heads(const void* in, int32_t in_ld, int32_t in_hs, int32_t in_off, void* out, int32_t out_ld, int32_t out_hs,
                                         int32_t out_off, int32_t n, int32_t H, const int64_t* positions, const float* freq_hi, const float* freq_lo,
-                                        int32_t pairs, float mag, int32_t T, int32_t dtype, int64_t stream) {
+                                        int32_t pairs, float mag, int32_t half, int32_t T, int32_t dtype, int64_t stream) {
   StkRotary r;
-  r.freq_hi = freq_hi, r.freq_lo = freq_lo, r.pairs = pairs, r.mag = mag;
+  r.freq_hi = freq_hi, r.freq_lo = freq_lo, r.pairs = pairs, r.mag = mag, r.half = half;
   vra_stack_rope_heads(in, in_ld, in_hs, in_off, out, out_ld, out_hs, out_off, n, H, positions, r, T, dtype, stream);
 }
 extern "C" void vra_stack_op_qk_norm_store(const float* raw, int32_t ld, int32_t nq, int32_t nk, int32_t nv, const float* q_w, const float* k_w, float eps,

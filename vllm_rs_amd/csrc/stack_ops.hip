@@ -1193,3 +1193,13 @@ extern "C" void vra_stack_op_attention(const void* q, int32_t ldq, void* out, co
   a.scale = scale, a.softcap = softcap, a.temp_coef = temp_coef, a.temp_every = temp_every;
   vra_stack_attention(a, dtype, stream);
 }
+// the matrix product with row groups and the element-wise epilogues: activation (epi 2), bias, soft cap
+extern "C" void vra_stack_op_gemm_post(const void* a, int32_t lda, const void* w, int64_t w_group_stride, void* out, int32_t ldo, int32_t out_f32, int32_t M,
+                                       int32_t N, int32_t K, float alpha, const float* bias, const int32_t* tile_group, int32_t granule, const int32_t* a_row,
+                                       const int32_t* out_row, int32_t epi, int32_t act, float softcap, int32_t dtype, int64_t stream) {
+  StkGemmArgs g;
+  g.a = a, g.lda = lda, g.w = w, g.w_group_stride = w_group_stride, g.out = out, g.ldo = ldo, g.out_f32 = out_f32, g.M = M, g.N = N, g.K = K;
+  g.alpha = alpha, g.bias = bias, g.tile_group = tile_group, g.granule = granule, g.a_row = a_row, g.out_row = out_row, g.epi = epi, g.act = act;
+  g.softcap = softcap;
+  vra_stack_gemm(g, dtype, stream);
+}
