@@ -180,9 +180,10 @@ def tensor_shapes(cfg):
     return out
 
 
-def random_tensors(cfg, seed):
+def random_tensors(cfg, seed, steady=False):
     """bfloat16-representable float32 tensors: projections ~ N(0, 1.5 / sqrt(fan in)), norm weights around one, layer scales spread over both
-    signs, corrections large enough to move the choice"""
+    signs, corrections large enough to move the choice.  steady: the corrections outweigh the scores' spread, so that few tokens stand before a
+    close call (a 16-bit model's rounding then turns few choices)"""
     r = np.random.default_rng(seed)
     out = {}
     for name, shape in tensor_shapes(cfg).items():
@@ -192,11 +193,11 @@ def random_tensors(cfg, seed):
         elif last in ("ls1", "ls2"):
             a = 0.7 + 0.5 * r.standard_normal(shape)
         elif last == "correction":
-            a = 0.3 * r.standard_normal(shape)
+            a = (1.0 if steady else 0.5) * r.standard_normal(shape)
         elif last == "embed":
             a = r.standard_normal(shape) / float(cfg["embedding"]["scale"])
         elif last == "router":
-            a = 3.0 * r.standard_normal(shape) / math.sqrt(shape[-1])
+            a = (0.4 if steady else 2.0) * r.standard_normal(shape) / math.sqrt(shape[-1])
         else:
             a = 1.5 * r.standard_normal(shape) / math.sqrt(shape[-1])
         out[name] = bf16_round(np.asarray(a, np.float32))
