@@ -82,6 +82,147 @@ __device__ __forceinline__ float center_rows(float* xs, int W, int tid, float ep
   return 1.f / sqrtf(block_sum_256(s, red) / (float)W + eps);
 }
 
+// a lane's partner by DPP (row-local controls only)
+template <int CTRL>
+__device__ __forceinline__ float dpp_f32(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float wave_sum_dpp(float v) {
+  v += dpp_f32<0xB1>(v);
+  v += dpp_f32<0x4E>(v);
+  v += dpp_f32<0x141>(v);
+  v += dpp_f32<0x140>(v);
+  return vra_xor32_sum(vra_xor16_sum(v));
+}
+__device__ __forceinline__ float wave_max_dpp(float v) {
+  v = fmaxf(v, dpp_f32<0xB1>(v));
+  v = fmaxf(v, dpp_f32<0x4E>(v));
+  v = fmaxf(v, dpp_f32<0x141>(v));
+  v = fmaxf(v, dpp_f32<0x140>(v));
+  return vra_xor32_max(vra_xor16_max(v));
+}
+
+// the choice among a row's n_router logits in zs (LDS; [n_router] scores and [n_groups] group scores behind them), all NT threads of the workgroup
+template <int NT>
+__device__ void router_pick(const StkSandwichArgs& a, int t, float* zs) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int n = a.n_router;
+  if (a.router_kind == 0) {  // the `top` largest in turn (ties: the lower index); a picked logit leaves the list
+    if (tid != 0) return;
+    float zmax = 0.f, sum = 0.f;
+    for (int j = 0; j < a.top; j++) {
+      int best = 0;
+      float bz = zs[0];
+      for (int e = 1; e < n; e++)
+        if (zs[e] > bz) best = e, bz = zs[e];
+      zs[best] = -INFINITY;
+      if (j == 0) zmax = bz;  // (the first pick is the largest logit)
+      const float w = expf(bz - zmax);
+      a.pair_expert[(size_t)t * a.top + j] = best;
+      a.pair_weight[(size_t)t * a.top + j] = w;
+      sum += w;
+    }
+    const float inv = 1.f / sum;
+    for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] *= inv;
+    return;
+  }
+  // Scores over all outputs; corrected scores choose, restricted to the best groups; the plain scores weigh.  The outputs are spread
+  // over the lanes of wave 0 (their corrections are fetched side by side, not one after the other), the groups over the threads.
+  float* sc = zs + n;        // [n] scores
+  float* gs = zs + 2 * n;    // [n_groups]
+  const bool sig = a.router_kind == 2;
+  if (wave == 0 && sig) {
+    for (int e = lane; e < n; e += 64) {
+      const float sv = sigmoidf_(zs[e]);
+      sc[e] = sv;
+      zs[e] = sv + (a.router_bias ? a.router_bias[e] : 0.f);
+    }
+  } else if (wave == 0) {
+    float m = -INFINITY, sum = 0.f;
+    for (int e = lane; e < n; e += 64) m = fmaxf(m, zs[e]);
+    m = wave_max(m);
+    for (int e = lane; e < n; e += 64) {
+      const float ex = expf(zs[e] - m);
+      sc[e] = ex;
+      sum += ex;
+    }
+    const float inv = 1.f / wave_sum(sum);
+    for (int e = lane; e < n; e += 64) {
+      const float sv = sc[e] * inv;
+      sc[e] = sv;
+      zs[e] = sv + (a.router_bias ? a.router_bias[e] : 0.f);
+    }
+  }
+  __syncthreads();
+  if (a.n_groups > 1 && a.keep < a.n_groups) {  // (uniform over the workgroup)
+    const int per = n / a.n_groups;
+    for (int g = tid; g < a.n_groups; g += NT) {
+      float b = zs[g * per], b2 = -INFINITY;  // the two largest
+      for (int e = 1; e < per; e++) {
+        const float v = zs[g * per + e];
+        b2 = fmaxf(b2, fminf(b, v));
+        b = fmaxf(b, v);
+      }
+      gs[g] = sig && per > 1 ? b + b2 : b;
+    }
+    __syncthreads();
+    for (int g = tid; g < a.n_groups; g += NT) {  // a group stays if fewer than `keep` groups come before it (larger score, or equal and lower index)
+      int before = 0;
+      for (int o = 0; o < a.n_groups; o++) before += (gs[o] > gs[g] || (gs[o] == gs[g] && o < g)) ? 1 : 0;
+      if (before >= a.keep)
+        for (int e = 0; e < per; e++) zs[g * per + e] = -INFINITY;
+    }
+    __syncthreads();
+  }
+  const int n_real = n - a.n_identity;
+  if (n <= 64) {  // one output a lane: a pick is a wave maximum and the lowest lane that holds it
+    if (wave != 0) return;
+    const bool have = lane < n;
+    const float val = have ? zs[lane] : 0.f, sv = have ? sc[lane] : 0.f;
+    bool avail = have;
+    float idw = 0.f, sum = 0.f, pick_w = 0.f;
+    int pick_e = -1;  // (lane j keeps pick j: top <= n <= 64)
+    for (int j = 0; j < a.top; j++) {
+      const float v = avail ? val : -INFINITY;
+      const float m = wave_max_dpp(v);
+      const unsigned long long holders = __ballot(avail && v == m);  // (left-out groups hold -inf: still chosen, in index order, once nothing else is left)
+      const int best = __ffsll((long long)holders) - 1;
+      const float w = __shfl(sv, best, 64);
+      if (lane == best) avail = false;
+      const bool ident = best >= n_real;
+      if (lane == j) pick_e = ident ? -1 : best, pick_w = w;
+      if (ident) idw += w;
+      sum += w;
+    }
+    const float norm = sig ? sum + 1e-20f : 1.f;
+    if (lane < a.top) {
+      a.pair_expert[(size_t)t * a.top + lane] = pick_e;
+      a.pair_weight[(size_t)t * a.top + lane] = sig ? pick_w / norm : pick_w;
+    }
+    if (lane == 0 && a.id_weight) a.id_weight[t] = idw / norm;
+    return;
+  }
+  if (tid != 0) return;
+  float idw = 0.f, sum = 0.f;
+  for (int j = 0; j < a.top; j++) {
+    int best = -1;
+    float bz = -INFINITY;
+    for (int e = 0; e < n; e++)
+      if (sc[e] >= 0.f && (best < 0 || zs[e] > bz)) best = e, bz = zs[e];
+    const float w = sc[best];
+    sc[best] = -1.f;  // (picked: out of the list)
+    const bool ident = best >= n_real;
+    a.pair_expert[(size_t)t * a.top + j] = ident ? -1 : best;
+    a.pair_weight[(size_t)t * a.top + j] = w;
+    if (ident) idw += w;
+    sum += w;
+  }
+  if (sig)
+    for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] /= sum + 1e-20f;
+  if (a.id_weight) a.id_weight[t] = sig ? idw / (sum + 1e-20f) : idw;
+}
+
+// any width
 template <typename T>
 __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   extern __shared__ float lds[];
@@ -212,120 +353,241 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
     }
   }
   __syncthreads();
-  const int n = a.n_router;
-  if (a.router_kind == 0) {  // the `top` largest in turn (ties: the lower index); a picked logit leaves the list
-    if (tid != 0) return;
-    float zmax = 0.f, sum = 0.f;
-    for (int j = 0; j < a.top; j++) {
-      int best = 0;
-      float bz = zs[0];
-      for (int e = 1; e < n; e++)
-        if (zs[e] > bz) best = e, bz = zs[e];
-      zs[best] = -INFINITY;
-      if (j == 0) zmax = bz;  // (the first pick is the largest logit)
-      const float w = expf(bz - zmax);
-      a.pair_expert[(size_t)t * a.top + j] = best;
-      a.pair_weight[(size_t)t * a.top + j] = w;
-      sum += w;
-    }
-    const float inv = 1.f / sum;
-    for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] *= inv;
-    return;
+  router_pick<256>(a, t, zs);
+}
+
+// The same seam for widths of whole 16-byte groups: a thread holds its columns (tid + v NT) * 4 .. + 3 in registers from the first load to the last
+// store, every operand of a sub-block is requested before the first sum needs one, a sum over the row costs one meeting, and (few rows,
+// 16-bit models) the first router rows are on their way while the norms run.
+template <int NW>
+__device__ __forceinline__ float row_sum(float v, float* red) {  // red: NW floats nobody else uses in this launch
+  v = wave_sum_dpp(v);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = 0.f;
+#pragma unroll
+  for (int w = 0; w < NW; w += 4) {
+    const float4 r = *(const float4*)(red + w);
+    s += (r.x + r.y) + (r.z + r.w);
   }
-  // Scores over all outputs; corrected scores choose, restricted to the best groups; the plain scores weigh.  The outputs are spread
-  // over the lanes of wave 0 (their corrections are fetched side by side, not one after the other), the groups over the threads.
-  float* sc = zs + n;        // [n] scores
-  float* gs = zs + 2 * n;    // [n_groups]
-  const bool sig = a.router_kind == 2;
-  if (wave == 0 && sig) {
-    for (int e = lane; e < n; e += 64) {
-      const float sv = sigmoidf_(zs[e]);
-      sc[e] = sv;
-      zs[e] = sv + (a.router_bias ? a.router_bias[e] : 0.f);
+  return s;
+}
+__device__ __forceinline__ float4 ld4(const float* p, bool in) { return in ? *(const float4*)p : make_float4(0.f, 0.f, 0.f, 0.f); }
+__device__ __forceinline__ float dot4(const float4& v, float s) { return fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, s)))); }
+
+template <typename T, int NT, int NV, int EB>
+__global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
+  constexpr int NW = NT / 64, NI = 8;
+  constexpr bool PREF = sizeof(T) == 2 && NT == 1024 && NV == 1;  // rows up to 8 * 512 columns
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ __attribute__((aligned(16))) float red[6][NW];
+  const int t = blockIdx.x, W = a.W, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  float* xs = lds;
+  float* zs = lds + W;
+  float* x = a.x + (size_t)t * W;
+  bool in[NV];
+  int col[NV];
+#pragma unroll
+  for (int v = 0; v < NV; v++) {
+    col[v] = (tid + v * NT) * 4;
+    in[v] = col[v] < W;
+    if (!in[v]) col[v] = 0;
+  }
+  float4 xv[NV];
+#pragma unroll
+  for (int v = 0; v < NV; v++) xv[v] = ld4(x + col[v], in[v]);
+  const T* rw = (const T*)a.router_w;
+  const bool vec8 = sizeof(T) == 2 && W % 8 == 0 && ((uintptr_t)rw % 16) == 0;  // 8 weights a load
+  u32x4 rp[PREF ? EB : 1][PREF ? NI : 1];
+  auto request_router = [&](int e0) {
+    if (PREF) {
+#pragma unroll
+      for (int i = 0; i < NI; i++)
+#pragma unroll
+        for (int u = 0; u < EB; u++) {
+          const int c = i * 512 + lane * 8;
+          rp[PREF ? u : 0][PREF ? i : 0] = *(const u32x4*)((const uint16_t*)rw + (size_t)min(e0 + u, a.n_router - 1) * W + (c < W ? c : 0));
+        }
     }
-  } else if (wave == 0) {
-    float m = -INFINITY, sum = 0.f;
-    for (int e = lane; e < n; e += 64) m = fmaxf(m, zs[e]);
-    m = wave_max(m);
-    for (int e = lane; e < n; e += 64) {
-      const float ex = expf(zs[e] - m);
-      sc[e] = ex;
-      sum += ex;
+  };
+  if (a.post_w) {
+    float4 s[NV], p2[NV], gw[NV];
+#pragma unroll
+    for (int v = 0; v < NV; v++) {
+      gw[v] = ld4(a.post_w + col[v], in[v]);
+      p2[v] = ld4(a.p2 ? a.p2 + (size_t)t * W + col[v] : x, in[v] && a.p2);
+      s[v] = make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    const float inv = 1.f / wave_sum(sum);
-    for (int e = lane; e < n; e += 64) {
-      const float sv = sc[e] * inv;
-      sc[e] = sv;
-      zs[e] = sv + (a.router_bias ? a.router_bias[e] : 0.f);
+    const float w2 = a.c2 * (a.p2w ? a.p2w[t] : 1.f);
+    if (a.n1 == 1 && !a.pw && !a.pe) {
+#pragma unroll
+      for (int v = 0; v < NV; v++) s[v] = ld4(a.p1 + (size_t)t * W + col[v], in[v]);
+    } else {
+      for (int j = 0; j < a.n1; j += 2) {  // two rows' requests at a time; a pair without a row (or beyond the last) counts as zeros
+        float4 r[2][NV];
+        float w[2];
+        bool ok[2];
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+          const size_t row = (size_t)t * a.n1 + min(j + u, a.n1 - 1);
+          ok[u] = j + u < a.n1 && !(a.pe && a.pe[row] < 0);
+          w[u] = a.pw ? a.pw[row] : 1.f;
+#pragma unroll
+          for (int v = 0; v < NV; v++) r[u][v] = *(const float4*)(a.p1 + row * W + col[v]);
+        }
+#pragma unroll
+        for (int u = 0; u < 2; u++)
+#pragma unroll
+          for (int v = 0; v < NV; v++) {
+            const bool k = ok[u] && in[v];
+            s[v].x = k ? fmaf(w[u], r[u][v].x, s[v].x) : s[v].x, s[v].y = k ? fmaf(w[u], r[u][v].y, s[v].y) : s[v].y;
+            s[v].z = k ? fmaf(w[u], r[u][v].z, s[v].z) : s[v].z, s[v].w = k ? fmaf(w[u], r[u][v].w, s[v].w) : s[v].w;
+          }
+      }
+    }
+    if (PREF && a.router_w && vec8) request_router(wave * EB);
+    auto part_norm = [&](float4* p, const float* nw, float* slot) {  // a part with an RMS norm of its own
+      float q = 0.f;
+#pragma unroll
+      for (int v = 0; v < NV; v++) q = dot4(p[v], q);
+      const float r = 1.f / sqrtf(row_sum<NW>(q, slot) / (float)W + a.eps);
+#pragma unroll
+      for (int v = 0; v < NV; v++) {
+        const float4 n = ld4(nw + col[v], in[v]);
+        p[v].x *= r * n.x, p[v].y *= r * n.y, p[v].z *= r * n.z, p[v].w *= r * n.w;
+      }
+    };
+    if (a.p1_norm_w) part_norm(s, a.p1_norm_w, red[0]);
+    if (a.p2 && a.p2_norm_w) part_norm(p2, a.p2_norm_w, red[1]);
+#pragma unroll
+    for (int v = 0; v < NV; v++) {
+      s[v].x = fmaf(w2, p2[v].x, s[v].x * a.c1), s[v].y = fmaf(w2, p2[v].y, s[v].y * a.c1);
+      s[v].z = fmaf(w2, p2[v].z, s[v].z * a.c1), s[v].w = fmaf(w2, p2[v].w, s[v].w * a.c1);
+    }
+    if (a.norm_kind == 1) {
+#pragma unroll
+      for (int v = 0; v < NV; v++) {
+        const float4 b = ld4(a.post_b + col[v], in[v]);
+        xv[v].x += tanhf(a.post_alpha * s[v].x) * gw[v].x + b.x, xv[v].y += tanhf(a.post_alpha * s[v].y) * gw[v].y + b.y;
+        xv[v].z += tanhf(a.post_alpha * s[v].z) * gw[v].z + b.z, xv[v].w += tanhf(a.post_alpha * s[v].w) * gw[v].w + b.w;
+      }
+    } else {
+      if (a.norm_kind == 2) {
+        float q = 0.f;
+#pragma unroll
+        for (int v = 0; v < NV; v++) q += (s[v].x + s[v].y) + (s[v].z + s[v].w);
+        const float mean = row_sum<NW>(q, red[2]) / (float)W;
+#pragma unroll
+        for (int v = 0; v < NV; v++)
+          if (in[v]) s[v].x -= mean, s[v].y -= mean, s[v].z -= mean, s[v].w -= mean;
+      }
+      float q = 0.f;
+#pragma unroll
+      for (int v = 0; v < NV; v++) q = dot4(s[v], q);
+      const float r = 1.f / sqrtf(row_sum<NW>(q, red[3]) / (float)W + a.eps);
+#pragma unroll
+      for (int v = 0; v < NV; v++) {
+        xv[v].x += s[v].x * r * gw[v].x, xv[v].y += s[v].y * r * gw[v].y;
+        xv[v].z += s[v].z * r * gw[v].z, xv[v].w += s[v].w * r * gw[v].w;
+      }
+    }
+#pragma unroll
+    for (int v = 0; v < NV; v++)
+      if (in[v]) *(float4*)(x + col[v]) = xv[v];
+  } else if (PREF && a.router_w && vec8) {
+    request_router(wave * EB);
+  }
+  if (!a.pre_w) return;
+  float r = 1.f;
+  if (a.norm_kind == 2) {
+    float q = 0.f;
+#pragma unroll
+    for (int v = 0; v < NV; v++) q += (xv[v].x + xv[v].y) + (xv[v].z + xv[v].w);
+    const float mean = row_sum<NW>(q, red[4]) / (float)W;
+#pragma unroll
+    for (int v = 0; v < NV; v++)
+      if (in[v]) xv[v].x -= mean, xv[v].y -= mean, xv[v].z -= mean, xv[v].w -= mean;
+  }
+  if (a.norm_kind != 1) {
+    float q = 0.f;
+#pragma unroll
+    for (int v = 0; v < NV; v++) q = dot4(xv[v], q);
+    r = 1.f / sqrtf(row_sum<NW>(q, red[5]) / (float)W + a.eps);
+  }
+  T* h = (T*)a.h + (size_t)t * W;
+#pragma unroll
+  for (int v = 0; v < NV; v++) {
+    if (!in[v]) continue;
+    const float4 g = *(const float4*)(a.pre_w + col[v]);
+    float4 y;
+    if (a.norm_kind == 1) {
+      const float4 b = *(const float4*)(a.pre_b + col[v]);
+      y.x = tanhf(a.pre_alpha * xv[v].x) * g.x + b.x, y.y = tanhf(a.pre_alpha * xv[v].y) * g.y + b.y;
+      y.z = tanhf(a.pre_alpha * xv[v].z) * g.z + b.z, y.w = tanhf(a.pre_alpha * xv[v].w) * g.w + b.w;
+    } else {
+      y.x = xv[v].x * r * g.x, y.y = xv[v].y * r * g.y, y.z = xv[v].z * r * g.z, y.w = xv[v].w * r * g.w;
+    }
+    if constexpr (sizeof(T) == 2) {
+      uint2 o;
+      o.x = BF16::pack2(y.x, y.y), o.y = BF16::pack2(y.z, y.w);
+      *(uint2*)(h + col[v]) = o;
+    } else {
+      *(float4*)(h + col[v]) = y;
+    }
+    if (a.h32) *(float4*)(a.h32 + (size_t)t * W + col[v]) = y;
+    if (a.router_w) *(float4*)(xs + col[v]) = y;
+  }
+  if (!a.router_w) return;
+  __syncthreads();
+  // a wave takes EB outputs at a time.  An output's sum keeps one order: a lane's columns ascending, then the lanes.
+  bool first = true;
+  for (int e0 = wave * EB; e0 < a.n_router; e0 += NW * EB) {
+    float z[EB];
+#pragma unroll
+    for (int u = 0; u < EB; u++) z[u] = 0.f;
+    auto add8 = [&](float& zu, const u32x4& v, int c) {
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        zu = fmaf(xs[c + 2 * i], __uint_as_float(v[i] << 16), zu);
+        zu = fmaf(xs[c + 2 * i + 1], __uint_as_float(v[i] & 0xffff0000u), zu);
+      }
+    };
+    if (PREF && vec8) {
+      if (!first) request_router(e0);
+#pragma unroll
+      for (int i = 0; i < NI; i++) {
+        const int c = i * 512 + lane * 8;
+        if (c < W)
+#pragma unroll
+          for (int u = 0; u < EB; u++) add8(z[u], rp[PREF ? u : 0][PREF ? i : 0], c);
+      }
+    } else if (vec8) {
+      for (int c = lane * 8; c < W; c += 512) {
+        u32x4 v[EB];
+#pragma unroll
+        for (int u = 0; u < EB; u++) v[u] = *(const u32x4*)((const uint16_t*)rw + (size_t)min(e0 + u, a.n_router - 1) * W + c);
+#pragma unroll
+        for (int u = 0; u < EB; u++) add8(z[u], v[u], c);
+      }
+    } else {
+      for (int c = lane; c < W; c += 64) {
+        float wv[EB];
+#pragma unroll
+        for (int u = 0; u < EB; u++) wv[u] = El<T>::ld(rw + (size_t)min(e0 + u, a.n_router - 1) * W + c);
+#pragma unroll
+        for (int u = 0; u < EB; u++) z[u] = fmaf(xs[c], wv[u], z[u]);
+      }
+    }
+    first = false;
+#pragma unroll
+    for (int u = 0; u < EB; u++) {
+      const float zu = wave_sum_dpp(z[u]);
+      const int e = e0 + u;
+      if (lane == 0 && e < a.n_router) zs[e] = zu + (a.router_kind == 0 && a.router_bias ? a.router_bias[e] : 0.f);
     }
   }
   __syncthreads();
-  if (a.n_groups > 1 && a.keep < a.n_groups) {  // (uniform over the workgroup)
-    const int per = n / a.n_groups;
-    for (int g = tid; g < a.n_groups; g += 256) {
-      float b = zs[g * per], b2 = -INFINITY;  // the two largest
-      for (int e = 1; e < per; e++) {
-        const float v = zs[g * per + e];
-        b2 = fmaxf(b2, fminf(b, v));
-        b = fmaxf(b, v);
-      }
-      gs[g] = sig && per > 1 ? b + b2 : b;
-    }
-    __syncthreads();
-    for (int g = tid; g < a.n_groups; g += 256) {  // a group stays if fewer than `keep` groups come before it (larger score, or equal and lower index)
-      int before = 0;
-      for (int o = 0; o < a.n_groups; o++) before += (gs[o] > gs[g] || (gs[o] == gs[g] && o < g)) ? 1 : 0;
-      if (before >= a.keep)
-        for (int e = 0; e < per; e++) zs[g * per + e] = -INFINITY;
-    }
-    __syncthreads();
-  }
-  const int n_real = n - a.n_identity;
-  if (n <= 64) {  // one output a lane: a pick is a wave maximum and the lowest lane that holds it
-    if (wave != 0) return;
-    const bool have = lane < n;
-    const float val = have ? zs[lane] : 0.f, sv = have ? sc[lane] : 0.f;
-    bool avail = have;
-    float idw = 0.f, sum = 0.f, pick_w = 0.f;
-    int pick_e = -1;  // (lane j keeps pick j: top <= n <= 64)
-    for (int j = 0; j < a.top; j++) {
-      const float v = avail ? val : -INFINITY;
-      const float m = wave_max(v);
-      const unsigned long long holders = __ballot(avail && v == m);  // (left-out groups hold -inf: still chosen, in index order, once nothing else is left)
-      const int best = __ffsll((long long)holders) - 1;
-      const float w = __shfl(sv, best, 64);
-      if (lane == best) avail = false;
-      const bool ident = best >= n_real;
-      if (lane == j) pick_e = ident ? -1 : best, pick_w = w;
-      if (ident) idw += w;
-      sum += w;
-    }
-    const float norm = sig ? sum + 1e-20f : 1.f;
-    if (lane < a.top) {
-      a.pair_expert[(size_t)t * a.top + lane] = pick_e;
-      a.pair_weight[(size_t)t * a.top + lane] = sig ? pick_w / norm : pick_w;
-    }
-    if (lane == 0 && a.id_weight) a.id_weight[t] = idw / norm;
-    return;
-  }
-  if (tid != 0) return;
-  float idw = 0.f, sum = 0.f;
-  for (int j = 0; j < a.top; j++) {
-    int best = -1;
-    float bz = -INFINITY;
-    for (int e = 0; e < n; e++)
-      if (sc[e] >= 0.f && (best < 0 || zs[e] > bz)) best = e, bz = zs[e];
-    const float w = sc[best];
-    sc[best] = -1.f;  // (picked: out of the list)
-    const bool ident = best >= n_real;
-    a.pair_expert[(size_t)t * a.top + j] = ident ? -1 : best;
-    a.pair_weight[(size_t)t * a.top + j] = w;
-    if (ident) idw += w;
-    sum += w;
-  }
-  if (sig)
-    for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] /= sum + 1e-20f;
-  if (a.id_weight) a.id_weight[t] = sig ? idw / (sum + 1e-20f) : idw;
+  router_pick<NT>(a, t, zs);
 }
 
 // ------------------------------------------------------------------------------------------------ per-head norm, rotary, cache rows
@@ -454,10 +716,6 @@ __global__ __launch_bounds__(256) void stk_sigmoid_pow_kernel(const float* z, in
 // sum over the P neighbouring lanes that share a column (P a power of two, lanes aligned to P), left in all of them.  Inside a row of 16
 // lanes the partner comes by DPP (quad permutes, then mirrors of half a row and of a row: after each step the lanes of a group hold one
 // value, so a mirror is as good as an xor); beyond 16 lanes by a cross-lane read.  One fixed order for a given P.
-template <int CTRL>
-__device__ __forceinline__ float dpp_f32(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false));
-}
 template <int P>
 __device__ __forceinline__ float group_sum(float v) {
   if (P >= 2) v += dpp_f32<0xB1>(v);    // quad_perm [1, 0, 3, 2]
@@ -807,6 +1065,30 @@ void vra_stack_sandwich_norm(const StkSandwichArgs& a, int dtype, int64_t stream
                 "stack seam norm: router groups / identity experts");
   const size_t lds = ((size_t)a.W + 2 * (size_t)a.n_router + (size_t)std::max(a.n_groups, 0) + 1) * sizeof(float);
   VRA_CHECK_ARG(lds <= 64 * 1024, "stack seam norm: row does not fit LDS");
+  hipStream_t st = as_stream(stream);
+  auto al16 = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  if (a.W % 4 == 0 && a.W <= 8192 && al16(a.x) && al16(a.p1) && al16(a.p2) && al16(a.post_w) && al16(a.post_b) && al16(a.pre_w) && al16(a.pre_b) && al16(a.h) &&
+      al16(a.h32) && al16(a.p1_norm_w) && al16(a.p2_norm_w)) {
+#define STK_SEAM(NTV, NVV, EBV)                                                                                                              \
+  do {                                                                                                                                       \
+    if (dtype == VRA_F32) launch_checked("stack seam norm", [&] { stk_seam_vec_kernel<float, NTV, NVV, EBV><<<a.T, NTV, lds, st>>>(a); });    \
+    else launch_checked("stack seam norm", [&] { stk_seam_vec_kernel<uint16_t, NTV, NVV, EBV><<<a.T, NTV, lds, st>>>(a); });                  \
+  } while (0)
+    if (a.T <= 256) {  // a row is a workgroup: few rows take many threads each
+      if (a.W <= 4096) STK_SEAM(1024, 1, 2);
+      else STK_SEAM(1024, 2, 2);
+    } else if (a.W <= 1024) {
+      STK_SEAM(256, 1, 4);
+    } else if (a.W <= 2048) {
+      STK_SEAM(256, 2, 4);
+    } else if (a.W <= 4096) {
+      STK_SEAM(256, 4, 4);
+    } else {
+      STK_SEAM(256, 8, 4);
+    }
+#undef STK_SEAM
+    return;
+  }
   if (dtype == VRA_F32) launch_checked("stack seam norm", [&] { stk_sandwich_kernel<float><<<a.T, 256, lds, as_stream(stream)>>>(a); });
   else launch_checked("stack seam norm", [&] { stk_sandwich_kernel<uint16_t><<<a.T, 256, lds, as_stream(stream)>>>(a); });
 }
