@@ -313,7 +313,52 @@ def parse_pesivik(cfg_json, dtype=None):
                 rms_norm_eps=float(norm.get("eps", 1e-5)), rope_theta=10000.0, dtype=dt, quant_method=None, spec="\n".join(lines) + "\n")
 
 
-STACK_ARCHS = {"Ditilix": parse_ditilix, "Gaperax": parse_gaperax, "Zifetar": parse_zifetar, "Sudosun": parse_sudosun, "Pesivik": parse_pesivik}
+def parse_kemavik(cfg_json, dtype=None):
+    """Kemavik config.json -> cfg dict with arch "stack": blocks that read the residual stream itself and norm only a sub-block's output (RMS norm,
+    weights stored around zero), per layer differential softmax attention (two maps over the same values, biases, per-head q / k norm, no
+    rotation, optionally another layer's keys and values) or time mixing with a matrix state (token shift, low-rank decays, bonus), and a
+    feed-forward that is dense (squared relu), a mixture of experts (softmax over all router outputs, a correction for the choice, identity
+    experts, a constant on the weights, a shared expert) or absent.  Every size and constant comes from the config; the rank of the decays'
+    projections comes from the tensors' shapes ("rank" of a mixer only sizes synthetic weights)."""
+    td = dtype or cfg_json.get("torch_dtype", "bfloat16")
+    dt = {"bfloat16": BF16, "bf16": BF16, "float32": F32, "f32": F32, BF16: BF16, F32: F32}.get(td)
+    if dt is None:
+        raise ValueError(f"dtype {td!r}: a layer stack runs in bfloat16 or float32")
+    norm = cfg_json.get("norm") or {}
+    width, vocab, layers = int(cfg_json["width"]), int(cfg_json["vocab"]), cfg_json["layers"]
+    lines = ["stack width=%d vocab=%d eps=%s block=post norm=rms pos=none norm_offset=1.0" % (width, vocab, _num(norm.get("eps", 1e-6)))]
+    heads = kv_heads = dim = 1
+    for i, layer in enumerate(layers):
+        mx, kind = layer["mixer"], layer.get("type")
+        if kind == "attention":
+            f = dict(mixer="differential", heads=int(mx["heads"]), kv_heads=int(mx.get("kv_heads", mx["heads"])), dim=int(mx["dim"]),
+                     vdim=int(mx.get("vdim", mx["dim"])), scale=_num(mx["scale"]) if mx.get("scale") is not None else _num(int(mx["dim"]) ** -0.5),
+                     diff=_num(mx["diff"]), kv_from=int(mx["kv_from"]) if mx.get("kv_from") is not None else -1)
+        elif kind == "wkv":
+            f = dict(mixer="wkv", heads=int(mx["heads"]), dim=int(mx["dim"]), rank_a=int(mx.get("rank", 32)))
+        else:
+            raise ValueError(f"layer {i}: mixer type {kind!r} is not part of this design")
+        mlp = layer.get("mlp")
+        if not mlp:
+            f.update(mlp="none")
+        elif mlp["kind"] == "dense":
+            f.update(mlp="relu2", ff=int(mlp["ff"]))
+        elif mlp["kind"] == "moe":
+            r = mlp["router"]
+            f.update(mlp="moe", ff=int(mlp["expert"]["ff"]), experts=int(r["experts"]), top=int(r.get("top", 1)), router="softmax_all", act="silu",
+                     identity=int(r.get("identity") or 0), router_scale=_num(r["scale"] if r.get("scale") is not None else 1.0))
+            if mlp.get("shared"):
+                f.update(shared_ff=int(mlp["shared"]["ff"]))
+        else:
+            raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not part of this design")
+        lines.append("layer " + " ".join(f"{k}={v}" for k, v in f.items()))
+        heads, kv_heads, dim = max(heads, f["heads"]), max(kv_heads, f.get("kv_heads", f["heads"])), max(dim, f["dim"], f.get("vdim", f["dim"]))
+    return dict(arch="stack", design="Kemavik", hidden_size=width, vocab_size=vocab, num_layers=len(layers), num_heads=heads, num_kv_heads=kv_heads,
+                head_dim=dim, intermediate_size=0, max_position_embeddings=int(cfg_json.get("max_position_embeddings", 1 << 20)),
+                rms_norm_eps=float(norm.get("eps", 1e-6)), rope_theta=10000.0, dtype=dt, quant_method=None, spec="\n".join(lines) + "\n")
+
+
+STACK_ARCHS = {"Ditilix": parse_ditilix, "Gaperax": parse_gaperax, "Zifetar": parse_zifetar, "Sudosun": parse_sudosun, "Pesivik": parse_pesivik, "Kemavik": parse_kemavik}
 
 
 def parse_config(cfg_json, dtype=None):

@@ -13,7 +13,8 @@
 // epi 0: plain.  epi 1: gated pair — W holds gate and up rows interleaved in blocks of 16 (block 2b = gate rows 16b.., block 2b+1 =
 // up rows 16b..), N counts both; out gets N/2 columns of  g' * sigmoid(act_alpha * g') * (u' + 1),  g' = min(g, limit),
 // u' = clamp(u, -limit, limit)  (limit <= 0: no clamp).
-// epi 2: element-wise activation of a plain product: out = act(alpha * sum + bias), act 3: the exact gelu 0.5 z (1 + erf(z / sqrt 2)).
+// epi 2: element-wise activation of a plain product: out = act(alpha * sum + bias), act 3: the exact gelu 0.5 z (1 + erf(z / sqrt 2)),
+// 4: max(z, 0)^2, 5: tanh z, 6: exp(-exp z) (a decay from its double logarithm).
 // softcap > 0 (plain products): out = softcap * tanh(v / softcap) of the finished value v.
 struct StkGemmArgs {
   const void* a = nullptr;
@@ -32,7 +33,7 @@ struct StkGemmArgs {
   const int* out_row = nullptr;
   int epi = 0;
   float limit = 0.f, act_alpha = 1.702f;
-  int act = 0;                  // the gated pair of epi 1: 0 the clamped form above, 1  gelu_tanh(g) * u, 2  silu(g) * u;  epi 2: 3 exact gelu
+  int act = 0;                  // the gated pair of epi 1: 0 the clamped form above, 1  gelu_tanh(g) * u, 2  silu(g) * u;  epi 2: 3 exact gelu, 4 squared relu, 5 tanh, 6 exp(-exp z)
   float softcap = 0.f;
   const float* bias = nullptr;  // f32 [N], added after alpha (plain epilogue)
   // batched form (no row groups): product z of `batch` reads a + z * a_batch_stride, w + z * w_batch_stride and writes out + z * out_batch_stride
@@ -113,6 +114,12 @@ struct StkAttnArgs {
   const float* head_scale = nullptr;  // f32 [H]: head h's scores are also multiplied by head_scale[h] (the sink is not)
   const float* gate = nullptr;  // f32 [T, gate_ld], column h: head h's output row is multiplied by sigmoid(gate[t, h])
   int gate_ld = 0;
+  // Differential form (maps = 2): q rows hold [map 1 | map 2] of `dim` values per query head, K rows the same per key/value head (k_ld 0: G * 2 *
+  // dim); each map is an attention of its own over the same values, a1 and a2 their outputs:
+  //   o = a1 - diff_lambda * a2,   out = o / sqrt(mean(o^2) + diff_eps) * diff_scale   (mean over the head's vdim values)
+  // everything up to the store in f32.  Causal mask, scale and sizes as above; no sink, gate, chunk, window, cap or temperature beside it.
+  int maps = 1;
+  float diff_lambda = 0.f, diff_eps = 0.f, diff_scale = 1.f;
   // latent decode form: f32 scratch of B * splits * H * (vdim + 2) floats for the parts of the key range (null: the one-launch kernel)
   float* scratch = nullptr;
   size_t scratch_bytes = 0;
@@ -238,8 +245,10 @@ void vra_stack_embed_pair(const StkEmbedPairArgs& a, int dtype, int64_t stream);
 //   s = c1 * sum_{j < n1} pw[t * n1 + j] * p1[(t * n1 + j), :]  +  c2 * p2w[t] * p2[t, :]   (pw, p2w null: weights 1; p2 null: no second part;
 //                                                                                       pe: pairs with pe[t * n1 + j] < 0 have no row and are left out)
 //   with p1_norm_w / p2_norm_w (n1 = 1): each part is first divided by its root mean square over the row and multiplied by that weight
+//         + xw[t] * x[t, :]                                                                 (xw null: absent; x before the sum below)
 //   x[t] += N(s; post_w)                                                              (post_w null: nothing is added)
 //   h[t]  = N(x[t]; pre_w)  in dtype                                                  (pre_w null: no h);  h32: also the unrounded h (f32)
+//   pre_identity: h[t] = x[t] in dtype, no norm (sub-blocks that read the residual stream itself); the router reads x[t]
 // N by norm_kind: 0 RMS norm with a weight; 1 Dynamic Tanh  tanh(alpha v) w + b  with the slopes post_alpha / pre_alpha and offsets post_b /
 // pre_b; 2 layer norm  (v - mean) / sqrt(mean((v - mean)^2) + eps) * w  (no offset).
 // With router_w ([n_router, W] in dtype): z = router_w . h + router_bias on the unrounded h, the `top` largest (ties: the lower
@@ -247,7 +256,7 @@ void vra_stack_embed_pair(const StkEmbedPairArgs& a, int dtype, int64_t stream);
 // softmax over all n_router logits; the choice goes by score + router_bias (a correction that the weights do not carry) among the experts of
 // the `keep` groups (of n_groups equal groups of neighbours) whose largest corrected score is largest; weights = the chosen scores as they
 // are; the last n_identity router outputs are experts without tensors that hand their input back: their pairs get expert -1 and their
-// weights are summed into id_weight[t].  router_kind 2: as 1, but scores = sigmoid of each logit, a group's worth is the SUM of its two largest
+// weights are summed into id_weight[t]; all weights times weight_scale.  router_kind 2: as 1, but scores = sigmoid of each logit, a group's worth is the SUM of its two largest
 // corrected scores (a group of one: that score), and the weights are the chosen scores divided by (their sum + 1e-20).  All f32.
 struct StkSandwichArgs {
   float* x = nullptr;
@@ -278,6 +287,9 @@ struct StkSandwichArgs {
   float* h32 = nullptr;
   int router_kind = 0, n_groups = 0, keep = 0, n_identity = 0;
   float* id_weight = nullptr;
+  const float* xw = nullptr;   // [T]
+  int pre_identity = 0;
+  float weight_scale = 1.f;    // router_kind 1
 };
 void vra_stack_sandwich_norm(const StkSandwichArgs& a, int dtype, int64_t stream);
 
@@ -355,6 +367,9 @@ struct StkScanArgs {
   int ldd = 0;
   int decay_per_head = 0;  // 1: decay [T, ldd] holds ONE decay per head and token (column h) instead of one per key channel
   int act_silu = 0;        // 1: q, k and v pass silu on their way in (constant decays per head only)
+  // f32 [H, dim] (per-row decays per key channel, no delta rule): the output reads the state BEFORE this token's decay and update, and the token
+  // itself through the bonus:   o_t = (S + diag(bonus_h) k_t v_t^T)^T (q_scale q_t) ;  S <- diag(d_t) S + k_t v_t^T
+  const float* bonus = nullptr;
   const float* head_decay = nullptr;
   const float* beta = nullptr;
   int ldb = 0;
@@ -370,9 +385,26 @@ struct StkScanArgs {
 void vra_stack_linear_scan(const StkScanArgs& a, int64_t stream);
 
 // out[t, h * vdim + c] = o[t, h, c] / sqrt(mean_c(o^2) + eps) * w[c] * act(gate[t, h * vdim + c])   (w null: 1; gate null: no gate;
-// gate_act 1: silu, 2: sigmoid);  o f32 [T, H * vdim], out in dtype
+// gate_act 1: silu, 2: sigmoid; w_per_head 1: w[h * vdim + c], a weight per head);  o f32 [T, H * vdim], out in dtype
 void vra_stack_head_norm_gate(const float* o, const float* w, const float* gate, int gate_ld, int gate_act, float eps, void* out, int T, int H, int vdim,
-                              int dtype, int64_t stream);
+                              int dtype, int64_t stream, int w_per_head = 0);
+
+// Token shift: n mixes of every token's row with the row before it in its sequence,
+//   out[m, t, c] = x[t, c] + (x'[t, c] - x[t, c]) * mu[m, c],   m < n;   x' = the previous token's row
+// (x f32 [T, W], mu f32 [n, W], out [n, T, W] in dtype).  The row before a step's first one comes from shift_state [slots, W] (f32; zeros for a
+// sequence that starts), which then takes the sequence's last row.
+struct StkShiftArgs {
+  const float* x = nullptr;
+  const float* mu = nullptr;
+  int n = 0;
+  float* shift_state = nullptr;
+  const int64_t* positions = nullptr;
+  const uint32_t* cu_q = nullptr;
+  const int32_t* state_slots = nullptr;
+  void* out = nullptr;
+  int T = 0, B = 0, W = 0;
+};
+void vra_stack_token_shift(const StkShiftArgs& a, int dtype, int64_t stream);
 
 // ---------------------------------------------------------------------------------------------------------------------------------------
 // A short causal convolution over time per channel with its state, and a gated diagonal linear recurrence (stack_recurrent.hip)

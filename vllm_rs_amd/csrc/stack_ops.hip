@@ -7,6 +7,8 @@
 // of a step, on a row's place in the batch or on the pages it uses — so a token's result does not depend on how its prompt was cut.
 #include <math.h>
 
+#include <algorithm>
+
 #include "stack_common.cuh"
 #include "stack_launch.h"
 
@@ -16,7 +18,12 @@ __device__ __forceinline__ float gelu_tanh_(float z) { return 0.5f * z * (1.f + 
 __device__ __forceinline__ float gelu_erf_(float z) { return 0.5f * z * (1.f + erff(z * 0.7071067811865476f)); }
 // the finished value of a plain product: element-wise activation (epi 2), soft cap
 __device__ __forceinline__ float plain_value(const StkGemmArgs& g, float v) {
-  if (g.epi == 2) v = gelu_erf_(v);
+  if (g.epi == 2) {
+    if (g.act == 3) v = gelu_erf_(v);
+    else if (g.act == 4) v = v > 0.f ? v * v : 0.f;
+    else if (g.act == 5) v = tanhf(v);
+    else v = expf(-expf(v));
+  }
   if (g.softcap > 0.f) v = g.softcap * tanhf(v / g.softcap);
   return v;
 }
@@ -520,15 +527,16 @@ __device__ __forceinline__ float cap_score_fast(float s, float softcap) {
 // Portions of prompts (and whatever else shares their step): 16 query rows of one head per workgroup, 4 per wave; key tiles of KT
 // tokens staged once in LDS (f32) for all 16 rows; lane = key for the scores, lane = value channel for the weighted sum.
 // Tiles start at key 0 of the sequence and a row's running maximum / sum go tile by tile: the order does not depend on the portion.
+// MAPS 2: the differential form of StkAttnArgs (a query row and a key row hold two maps; both weigh the same staged values).
 #define STK_QT 16
-template <typename T, int KT, int NR>
+template <typename T, int KT, int NR, int MAPS>
 __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   extern __shared__ float lds[];
-  const int dim = a.dim, vdim = a.vdim, kld = dim + 1;
-  float* qs = lds;                      // [16][dim]  q * temp
-  float* ks = qs + STK_QT * dim;        // [KT][dim + 1]
+  const int dim = a.dim, vdim = a.vdim, dm = MAPS * dim, kld = dm + 1;
+  float* qs = lds;                      // [16][dm]  q * temp
+  float* ks = qs + STK_QT * dm;         // [KT][dm + 1]
   float* vs = ks + KT * kld;            // [KT][vdim]
-  float* ps = vs + KT * vdim;           // [16][KT]
+  float* ps = vs + KT * vdim;           // [MAPS][16][KT]
   const int b = blockIdx.y, h = blockIdx.z, g = h / (a.H / a.G);
   const int q0 = a.cu_q[b], q1 = a.cu_q[b + 1];
   const int t0 = q0 + blockIdx.x * STK_QT;
@@ -536,10 +544,10 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   const int nq = min(STK_QT, q1 - t0);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const T* q = (const T*)a.q;
-  for (int i = tid; i < STK_QT * dim; i += 256) {
-    const int r = i / dim, d = i % dim;
+  for (int i = tid; i < STK_QT * dm; i += 256) {
+    const int r = i / dm, d = i % dm;
     float v = 0.f;
-    if (r < nq) v = El<T>::ld(q + (size_t)(t0 + r) * a.ldq + h * dim + d) * q_temperature(a.positions[t0 + r], a.temp_coef, a.temp_every);
+    if (r < nq) v = El<T>::ld(q + (size_t)(t0 + r) * a.ldq + h * dm + d) * q_temperature(a.positions[t0 + r], a.temp_coef, a.temp_every);
     qs[i] = v;
   }
   int64_t pq[4], plo[4];
@@ -556,25 +564,26 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   for (int r = 0; r < nq; r++) pmax = max(pmax, a.positions[t0 + r]), lo_min = min(lo_min, block_start(a.positions[t0 + r]));
   const int n_keys = (int)min((int64_t)a.context_lens[b], pmax + 1);
   const int kt_begin = (int)(lo_min / KT) * KT;  // (tiles stay aligned to absolute positions)
-  float m[4], l[4], acc[4][NR];
-  for (int i = 0; i < 4; i++) {
-    m[i] = -INFINITY, l[i] = 0.f;
-    if (a.sink) m[i] = a.sink[h], l[i] = 1.f;  // the sink: one more term exp(sink - m) of the denominator, present from the start
-    for (int r = 0; r < NR; r++) acc[i][r] = 0.f;
-  }
+  float m[MAPS][4], l[MAPS][4], acc[MAPS][4][NR];
+  for (int mp = 0; mp < MAPS; mp++)
+    for (int i = 0; i < 4; i++) {
+      m[mp][i] = -INFINITY, l[mp][i] = 0.f;
+      if (a.sink) m[mp][i] = a.sink[h], l[mp][i] = 1.f;  // the sink: one more term exp(sink - m) of the denominator, present from the start
+      for (int r = 0; r < NR; r++) acc[mp][i][r] = 0.f;
+    }
   const T* kc = (const T*)a.kc;
   const T* vc = (const T*)a.vc;
   const uint32_t* bt = a.block_tables + (size_t)b * a.max_blocks;
-  const int kdim = a.k_ld ? a.k_ld : a.G * dim, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
+  const int kdim = a.k_ld ? a.k_ld : a.G * dm, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
   const float hscale = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
   for (int kt0 = kt_begin; kt0 < n_keys; kt0 += KT) {
     __syncthreads();
-    for (int i = tid; i < KT * dim; i += 256) {
-      const int j = i / dim, d = i % dim, key = kt0 + j;
+    for (int i = tid; i < KT * dm; i += 256) {
+      const int j = i / dm, d = i % dm, key = kt0 + j;
       float v = 0.f;
       if (key < n_keys) {
         const int64_t slot = (int64_t)bt[key / a.BS] * a.BS + key % a.BS;
-        v = El<T>::ld(kc + slot * kdim + g * dim + d);
+        v = El<T>::ld(kc + slot * kdim + g * dm + d);
       }
       ks[j * kld + d] = v;
     }
@@ -588,25 +597,26 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
       vs[i] = v;
     }
     __syncthreads();
-    for (int i = 0; i < 4; i++) {
-      const int r = wave * 4 + i;
-      float s = -INFINITY;
-      if (lane < KT && pq[i] >= 0 && kt0 + lane <= pq[i] && kt0 + lane >= plo[i] && kt0 + lane < n_keys) {
-        float d0 = 0.f;
-        for (int d = 0; d < dim; d++) d0 = fmaf(qs[r * dim + d], ks[lane * kld + d], d0);
-        s = cap_score(d0 * hscale, a.softcap);
+    for (int mp = 0; mp < MAPS; mp++)
+      for (int i = 0; i < 4; i++) {
+        const int r = wave * 4 + i;
+        float s = -INFINITY;
+        if (lane < KT && pq[i] >= 0 && kt0 + lane <= pq[i] && kt0 + lane >= plo[i] && kt0 + lane < n_keys) {
+          float d0 = 0.f;
+          for (int d = 0; d < dim; d++) d0 = fmaf(qs[r * dm + mp * dim + d], ks[lane * kld + mp * dim + d], d0);
+          s = cap_score(d0 * hscale, a.softcap);
+        }
+        const float mn = fmaxf(m[mp][i], wave_max(s));
+        float p = 0.f, corr = 1.f;
+        if (mn > -INFINITY) {
+          p = s > -INFINITY ? expf(s - mn) : 0.f;
+          corr = m[mp][i] > -INFINITY ? expf(m[mp][i] - mn) : 0.f;
+        }
+        l[mp][i] = l[mp][i] * corr + wave_sum(p);
+        m[mp][i] = mn;
+        for (int rr = 0; rr < NR; rr++) acc[mp][i][rr] *= corr;
+        if (lane < KT) ps[(mp * STK_QT + r) * KT + lane] = p;
       }
-      const float mn = fmaxf(m[i], wave_max(s));
-      float p = 0.f, corr = 1.f;
-      if (mn > -INFINITY) {
-        p = s > -INFINITY ? expf(s - mn) : 0.f;
-        corr = m[i] > -INFINITY ? expf(m[i] - mn) : 0.f;
-      }
-      l[i] = l[i] * corr + wave_sum(p);
-      m[i] = mn;
-      for (int rr = 0; rr < NR; rr++) acc[i][rr] *= corr;
-      if (lane < KT) ps[r * KT + lane] = p;
-    }
     __syncthreads();
     for (int rr = 0; rr < NR; rr++) {
       const int d = lane + 64 * rr;
@@ -614,7 +624,8 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
 #pragma unroll 4
       for (int j = 0; j < KT; j++) {
         const float v = vs[j * vdim + d];
-        for (int i = 0; i < 4; i++) acc[i][rr] = fmaf(ps[(wave * 4 + i) * KT + j], v, acc[i][rr]);
+        for (int mp = 0; mp < MAPS; mp++)
+          for (int i = 0; i < 4; i++) acc[mp][i][rr] = fmaf(ps[(mp * STK_QT + wave * 4 + i) * KT + j], v, acc[mp][i][rr]);
       }
     }
   }
@@ -622,11 +633,23 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
   for (int i = 0; i < 4; i++) {
     const int r = wave * 4 + i;
     if (r >= nq) continue;
-    float inv = l[i] > 0.f ? 1.f / l[i] : 0.f;
+    if constexpr (MAPS == 2) {
+      const float i1 = l[0][i] > 0.f ? 1.f / l[0][i] : 0.f, i2 = l[MAPS - 1][i] > 0.f ? a.diff_lambda / l[MAPS - 1][i] : 0.f;
+      float o[NR], q2 = 0.f;
+      for (int rr = 0; rr < NR; rr++) {
+        o[rr] = lane + 64 * rr < vdim ? acc[0][i][rr] * i1 - acc[MAPS - 1][i][rr] * i2 : 0.f;
+        q2 = fmaf(o[rr], o[rr], q2);
+      }
+      const float f = a.diff_scale / sqrtf(wave_sum(q2) / (float)vdim + a.diff_eps);
+      for (int rr = 0; rr < NR; rr++)
+        if (lane + 64 * rr < vdim) El<T>::st(out + (size_t)(t0 + r) * a.H * vdim + h * vdim + lane + 64 * rr, o[rr] * f);
+      continue;
+    }
+    float inv = l[0][i] > 0.f ? 1.f / l[0][i] : 0.f;
     if (a.gate) inv *= sigmoidf_(a.gate[(size_t)(t0 + r) * a.gate_ld + h]);
     for (int rr = 0; rr < NR; rr++) {
       const int d = lane + 64 * rr;
-      if (d < vdim) El<T>::st(out + (size_t)(t0 + r) * a.H * vdim + h * vdim + d, acc[i][rr] * inv);
+      if (d < vdim) El<T>::st(out + (size_t)(t0 + r) * a.H * vdim + h * vdim + d, acc[0][i][rr] * inv);
     }
   }
 }
@@ -640,18 +663,25 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
 //                   scores (position = oct * 8 + half * 4 + j), B = the lane's own 8 weights.  The weights stay f32 in effect: each is
 //                   split into a bf16 head and a bf16 tail (p = hi + lo to 2^-17) and the product runs twice.
 // Every sum goes tile by tile from key 0 with a fixed lane pattern: the result of a row does not depend on the portion it came in.
-template <int DC, int VT>
-__global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs a) {
+// MAPS 2: the differential form of StkAttnArgs.  Four more waves own the second map of the same 64 rows (their registers are those of the plain
+// kernel), all eight share the transposed V tile; at the end the second map's rows travel through LDS to the first map's waves, which
+// combine, norm and store.
+template <int DC, int VT, int MAPS>
+__global__ __launch_bounds__(256 * MAPS) void stk_attn_prefill_mfma_kernel(StkAttnArgs a) {
   constexpr int KT = 32, VLD = KT + 8;  // LDS row of a value channel: 32 positions + 8 (rows stay 16-byte aligned, lanes spread over banks)
-  __shared__ __attribute__((aligned(16))) uint16_t vt[VT * 16 * VLD];
-  const int dim = a.dim, vdim = a.vdim;
+  constexpr int NT = 256 * MAPS, XT = VT < 4 ? VT : 4;  // threads; channel tiles handed over at a time (MAPS 2: 4 waves x 64 lanes x 16 bytes each)
+  constexpr int VT_BYTES = VT * 16 * VLD * 2, X_BYTES = MAPS == 2 ? XT * 4096 : 0;
+  __shared__ __attribute__((aligned(16))) unsigned char smem[VT_BYTES > X_BYTES ? VT_BYTES : X_BYTES];
+  uint16_t* vt = (uint16_t*)smem;
+  const int dim = a.dim, vdim = a.vdim, dm = MAPS * dim;
   const int b = blockIdx.y, h = blockIdx.z, g = h / (a.H / a.G);
   const int q0 = a.cu_q[b], q1 = a.cu_q[b + 1];
   // the last row blocks of a portion see the most keys: they are dispatched first, so that no long block is left to run alone at the end
   const int t0 = q0 + ((int)gridDim.x - 1 - (int)blockIdx.x) * 64;
   if (t0 >= q1) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, rq = lane & 15, oct = lane >> 4;
-  const int tq = t0 + wave * 16 + rq;  // this lane's query row
+  const int mp = MAPS == 2 ? wave >> 2 : 0;  // this wave's map
+  const int tq = t0 + (wave & 3) * 16 + rq;  // this lane's query row
   const bool qv = tq < q1;
   const int64_t pq = qv ? a.positions[tq] : -1;
   const uint16_t* q = (const uint16_t*)a.q;
@@ -660,7 +690,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
   for (int c = 0; c < DC; c++) {
     const int ch = c * 32 + oct * 8;
     const bool ok = qv && ch < dim;
-    const u32x4 v = *(const u32x4*)(q + (size_t)(ok ? tq : q0) * a.ldq + h * dim + (ok ? ch : 0));
+    const u32x4 v = *(const u32x4*)(q + (size_t)(ok ? tq : q0) * a.ldq + h * dm + mp * dim + (ok ? ch : 0));
     qf[c] = ok ? v : zero4;
   }
   const float sc = a.scale * q_temperature(pq < 0 ? 0 : pq, a.temp_coef, a.temp_every) * (a.head_scale ? a.head_scale[h] : 1.f);
@@ -672,7 +702,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
   if (a.window > 0 && pq >= 0) key_lo = max(key_lo, pq - a.window + 1);
   int64_t lmin = pq >= 0 ? key_lo : INT64_MAX;
   for (int o = 32; o > 0; o >>= 1) lmin = min(lmin, (int64_t)__shfl_xor((long long)lmin, o, 64));
-  __shared__ long long wmax[4], wmin[4];
+  __shared__ long long wmax[4 * MAPS], wmin[4 * MAPS];  // (the waves of the second map own the same rows)
   if (lane == 0) wmax[wave] = pmax, wmin[wave] = lmin;
   __syncthreads();
   const int64_t gmax = max(max(wmax[0], wmax[1]), max(wmax[2], wmax[3]));
@@ -683,7 +713,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
   const uint16_t* kc = (const uint16_t*)a.kc;
   const uint16_t* vc = (const uint16_t*)a.vc;
   const uint32_t* bt = a.block_tables + (size_t)b * a.max_blocks;
-  const int kdim = a.k_ld ? a.k_ld : a.G * dim, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
+  const int kdim = a.k_ld ? a.k_ld : a.G * dm, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
   f32x4 acc[VT];
   for (int t = 0; t < VT; t++) acc[t] = vra_zero_acc();
   float m = -INFINITY, l = 0.f;
@@ -694,7 +724,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
   // The K fragments and this thread's share of the V tile are requested one tile ahead, so that their way from memory runs beside the
   // current tile's arithmetic.  V item = (key, 8 channels): NV per thread.
   // V item = (pair of neighbouring keys, 8 channels): NV per thread, two 16-byte requests each
-  constexpr int NV = (KT / 2 * VT * 2 + 255) / 256;
+  constexpr int NV = (KT / 2 * VT * 2 + NT - 1) / NT;
   u32x4 kfn[2][DC], vgn[NV][2];
   // The page size is a multiple of 32 (the launcher sends other sizes to the FMA kernel), so a 32-key tile lies in ONE page: its first
   // slot is a scalar, read from the block table one tile ahead of the requests that use it — no request of a tile waits behind a
@@ -709,7 +739,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
       const int key = kt0 + u * 16 + rq;
       const bool kv = key < n_keys;
       const int64_t slot = kv ? slot_of(key) : 0;
-      const uint16_t* kr = kc + slot * kdim + g * dim;
+      const uint16_t* kr = kc + slot * kdim + g * dm + mp * dim;
       for (int c = 0; c < DC; c++) {
         const int ch = c * 32 + oct * 8;
         const bool ok = kv && ch < dim;
@@ -718,7 +748,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
       }
     }
     for (int n = 0; n < NV; n++) {
-      const int i = tid + n * 256;
+      const int i = tid + n * NT;
       const int kp = i / (VT * 2), c8 = (i % (VT * 2)) * 8;
       for (int e = 0; e < 2; e++) {
         const int key = kt0 + kp * 2 + e;
@@ -740,7 +770,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
     // V tile -> LDS, transposed, the keys in the order the lanes hold their scores: keys 2 kp and 2 kp + 1 are neighbours there too,
     // so one 32-bit store carries both for a channel
     for (int n = 0; n < NV; n++) {
-      const int i = tid + n * 256;
+      const int i = tid + n * NT;
       if (i >= KT / 2 * VT * 2) break;
       const int kl = (i / (VT * 2)) * 2, c8 = (i % (VT * 2)) * 8;
       const int pos = ((kl & 15) >> 2) * 8 + (kl >> 4) * 4 + (kl & 3);  // even
@@ -817,6 +847,43 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
+  if constexpr (MAPS == 2) {  // (channels beyond vdim hold zeros: their V columns were staged as zeros)
+    const float inv = l > 0.f ? (mp == 0 ? 1.f : a.diff_lambda) / l : 0.f;
+    float* ex = (float*)smem;
+    float q2 = 0.f;
+#pragma unroll
+    for (int x0 = 0; x0 < VT; x0 += XT) {
+      __syncthreads();
+      if (mp == 1)
+#pragma unroll
+        for (int t = 0; t < XT; t++) *(f32x4*)(ex + ((t * 4 + (wave & 3)) * 64 + lane) * 4) = acc[x0 + t] * inv;
+      __syncthreads();
+      if (mp == 0)
+#pragma unroll
+        for (int t = 0; t < XT; t++) {
+          const f32x4 o2 = *(const f32x4*)(ex + ((t * 4 + wave) * 64 + lane) * 4);
+#pragma unroll
+          for (int j = 0; j < 4; j++) {
+            const float o = acc[x0 + t][j] * inv - o2[j];
+            acc[x0 + t][j] = o;
+            q2 = fmaf(o, o, q2);
+          }
+        }
+    }
+    q2 += __shfl_xor(q2, 16, 64);
+    q2 += __shfl_xor(q2, 32, 64);
+    if (mp == 1 || !qv) return;
+    const float f = a.diff_scale / sqrtf(q2 / (float)vdim + a.diff_eps);
+    uint16_t* out = (uint16_t*)a.out + (size_t)tq * a.H * vdim + h * vdim;
+#pragma unroll
+    for (int t = 0; t < VT; t++) {
+      const int c = t * 16 + oct * 4;  // (vdim is a multiple of 16: a lane's four channels are in or out together)
+      uint2 p;
+      p.x = BF16::pack2(acc[t][0] * f, acc[t][1] * f), p.y = BF16::pack2(acc[t][2] * f, acc[t][3] * f);
+      if (c < vdim) *(uint2*)(out + c) = p;
+    }
+    return;
+  }
   if (!qv) return;
   float inv = l > 0.f ? 1.f / l : 0.f;
   if (a.gate) inv *= sigmoidf_(a.gate[(size_t)tq * a.gate_ld + h]);
@@ -831,6 +898,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_mfma_kernel(StkAttnArgs 
 // One decoded token per sequence: a workgroup per (sequence, query head); its 8 waves take the 64-key tiles of the context in turn,
 // read K rows straight from the cache (lane = key, 16 bytes a load where the row allows) and V rows channel-wise (lane = channel), and
 // meet once in LDS.  The order of the sums depends on the context length alone.
+// MAPS 2: the differential form of StkAttnArgs (both maps' scores of a key, then one pass over the values for both).
 #define STK_DW 8
 template <typename T>
 __device__ __forceinline__ float stk_dot_row(const float* qs, const T* kr, int dim) {
@@ -854,36 +922,40 @@ __device__ __forceinline__ float stk_dot_row<uint16_t>(const float* qs, const ui
   for (int d = 0; d < dim; d++) d0 = fmaf(qs[d], BF16::to_f32(kr[d]), d0);
   return d0;
 }
-template <typename T, int NR>
+template <typename T, int NR, int MAPS>
 __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArgs a) {
   extern __shared__ float lds[];
-  const int dim = a.dim, vdim = a.vdim;
-  float* qs = lds;                     // [dim]
-  float* ps = qs + dim;                // [waves][64]
-  float* ms = ps + STK_DW * 64;        // [waves] max, [waves] sum
-  float* os = ms + 2 * STK_DW;         // [waves][vdim]
-  int* ss = (int*)(os + STK_DW * vdim);  // [waves][64] cache slot of each key of the wave's current tile
+  const int dim = a.dim, vdim = a.vdim, dm = MAPS * dim;
+  float* qs = lds;                     // [dm]
+  float* ps = qs + dm;                 // [MAPS][waves][64]
+  float* ms = ps + MAPS * STK_DW * 64;   // [MAPS][waves] max, [MAPS][waves] sum
+  float* os = ms + MAPS * 2 * STK_DW;    // [MAPS][waves][vdim]
+  int* ss = (int*)(os + MAPS * STK_DW * vdim);  // [waves][64] cache slot of each key of the wave's current tile
   const int b = blockIdx.x, h = blockIdx.y, g = h / (a.H / a.G);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int64_t p = a.positions[b];
   const int n_keys = (int)min((int64_t)a.context_lens[b], p + 1);
-  const T* q = (const T*)a.q + (size_t)b * a.ldq + h * dim;
+  const T* q = (const T*)a.q + (size_t)b * a.ldq + h * dm;
   const float temp = q_temperature(p, a.temp_coef, a.temp_every);
-  for (int d = tid; d < dim; d += 64 * STK_DW) qs[d] = El<T>::ld(q + d) * temp;
+  for (int d = tid; d < dm; d += 64 * STK_DW) qs[d] = El<T>::ld(q + d) * temp;
   __syncthreads();
   const T* kc = (const T*)a.kc;
   const T* vc = (const T*)a.vc;
   const uint32_t* bt = a.block_tables + (size_t)b * a.max_blocks;
-  const int kdim = a.k_ld ? a.k_ld : a.G * dim, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
-  float m = -INFINITY, l = 0.f, acc[NR];
-  for (int i = 0; i < NR; i++) acc[i] = 0.f;
-  if (a.sink && wave == 0) m = a.sink[h], l = 1.f;
+  const int kdim = a.k_ld ? a.k_ld : a.G * dm, vd_all = a.v_ld ? a.v_ld : a.G * vdim;
+  float m[MAPS], l[MAPS], acc[MAPS][NR], vacc[MAPS][8];
+#pragma unroll
+  for (int mp = 0; mp < MAPS; mp++) {
+    m[mp] = -INFINITY, l[mp] = 0.f;
+    for (int i = 0; i < NR; i++) acc[mp][i] = 0.f;
+    for (int i = 0; i < 8; i++) vacc[mp][i] = 0.f;
+  }
+  if (a.sink && wave == 0) m[0] = a.sink[h], l[0] = 1.f;
   // 16-bit values in whole octets: the value phase reads 16 bytes a lane (oc = channel octets rounded up to a power of two)
   const bool vec = sizeof(T) == 2 && vdim % 8 == 0 && vd_all % 8 == 0 && ((uintptr_t)vc % 16) == 0;
   int oc = 1;
   while (oc * 8 < vdim) oc <<= 1;
   const int co = lane & (oc - 1), kg = lane / oc, kpar = 64 / oc;
-  float vacc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   // block mask: the keys from key_lo on; tiles stay aligned to absolute positions (the first one may begin below key_lo: those keys
   // count with weight 0)
   int key_lo = a.chunk > 0 ? (int)(p / a.chunk * a.chunk) : 0;
@@ -891,18 +963,24 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
   const float hscale = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
   for (int kt0 = key_lo / 64 * 64 + wave * 64; kt0 < n_keys; kt0 += STK_DW * 64) {
     const int key = kt0 + lane;
-    float s = -INFINITY;
+    float s[MAPS], corr[MAPS];
+    for (int mp = 0; mp < MAPS; mp++) s[mp] = -INFINITY;
     if (key < n_keys) {
       const int64_t slot = (int64_t)bt[key / a.BS] * a.BS + key % a.BS;
       ss[wave * 64 + lane] = (int)slot;
-      if (key >= key_lo) s = cap_score(stk_dot_row<T>(qs, kc + slot * kdim + g * dim, dim) * hscale, a.softcap);
+      if (key >= key_lo)
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) s[mp] = cap_score(stk_dot_row<T>(qs + mp * dim, kc + slot * kdim + g * dm + mp * dim, dim) * hscale, a.softcap);
     }
-    const float mn = fmaxf(m, wave_max(s));  // (the tile's first key exists: mn is finite)
-    const float pj = s > -INFINITY ? expf(s - mn) : 0.f;
-    const float corr = m > -INFINITY ? expf(m - mn) : 0.f;
-    l = l * corr + wave_sum(pj);
-    m = mn;
-    ps[wave * 64 + lane] = pj;
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) {
+      const float mn = fmaxf(m[mp], wave_max(s[mp]));  // (the tile's first key exists: mn is finite)
+      const float pj = s[mp] > -INFINITY ? expf(s[mp] - mn) : 0.f;
+      corr[mp] = m[mp] > -INFINITY ? expf(m[mp] - mn) : 0.f;
+      l[mp] = l[mp] * corr[mp] + wave_sum(pj);
+      m[mp] = mn;
+      ps[(mp * STK_DW + wave) * 64 + lane] = pj;
+    }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
@@ -910,63 +988,91 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
     if (vec) {
       // lane = (key group kg, channel octet co): one 16-byte load covers 8 channels of one key, 64 / OC keys are in flight per step;
       // the groups' partial sums meet after the last tile
-      for (int i = 0; i < 8; i++) vacc[i] *= corr;
+#pragma unroll
+      for (int mp = 0; mp < MAPS; mp++)
+        for (int i = 0; i < 8; i++) vacc[mp][i] *= corr[mp];
       // four keys of a group per step, their rows requested together (the slots come from LDS, where the score phase left them, so no
       // request waits for a block-table read); keys beyond the tile count with weight 0
       for (int j = kg; j < nj && co * 8 < vdim; j += 4 * kpar) {
         u32x4 v[4];
-        float pw[4];
+        float pw[MAPS][4];
         for (int u = 0; u < 4; u++) {
           const int ju = j + u * kpar;
           const bool in = ju < nj;
           const int64_t sl = ss[wave * 64 + (in ? ju : j)];
           v[u] = *(const u32x4*)((const uint16_t*)vc + sl * vd_all + g * vdim + co * 8);
-          pw[u] = in ? ps[wave * 64 + ju] : 0.f;
+#pragma unroll
+          for (int mp = 0; mp < MAPS; mp++) pw[mp][u] = in ? ps[(mp * STK_DW + wave) * 64 + ju] : 0.f;
         }
         for (int u = 0; u < 4; u++)
-          for (int i = 0; i < 4; i++) {
-            vacc[2 * i] = fmaf(pw[u], __uint_as_float(v[u][i] << 16), vacc[2 * i]);
-            vacc[2 * i + 1] = fmaf(pw[u], __uint_as_float(v[u][i] & 0xffff0000u), vacc[2 * i + 1]);
-          }
+#pragma unroll
+          for (int mp = 0; mp < MAPS; mp++)
+            for (int i = 0; i < 4; i++) {
+              vacc[mp][2 * i] = fmaf(pw[mp][u], __uint_as_float(v[u][i] << 16), vacc[mp][2 * i]);
+              vacc[mp][2 * i + 1] = fmaf(pw[mp][u], __uint_as_float(v[u][i] & 0xffff0000u), vacc[mp][2 * i + 1]);
+            }
       }
     } else {
       for (int rr = 0; rr < NR; rr++) {
         const int d = lane + 64 * rr;
         if (d >= vdim) break;
-        float o = acc[rr] * corr;
-        for (int j = 0; j < nj; j++) o = fmaf(ps[wave * 64 + j], El<T>::ld(vc + (int64_t)ss[wave * 64 + j] * vd_all + g * vdim + d), o);
-        acc[rr] = o;
+        float o[MAPS];
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) o[mp] = acc[mp][rr] * corr[mp];
+        for (int j = 0; j < nj; j++) {
+          const float v = El<T>::ld(vc + (int64_t)ss[wave * 64 + j] * vd_all + g * vdim + d);
+#pragma unroll
+          for (int mp = 0; mp < MAPS; mp++) o[mp] = fmaf(ps[(mp * STK_DW + wave) * 64 + j], v, o[mp]);
+        }
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) acc[mp][rr] = o[mp];
       }
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
   }
-  if (vec) {
-    for (int o = oc; o < 64; o <<= 1)
-      for (int i = 0; i < 8; i++) vacc[i] += __shfl_xor(vacc[i], o, 64);
-    if (lane < oc && co * 8 < vdim)
-      for (int i = 0; i < 8; i++) os[wave * vdim + co * 8 + i] = vacc[i];
-  } else {
-    for (int rr = 0; rr < NR; rr++) {
-      const int d = lane + 64 * rr;
-      if (d < vdim) os[wave * vdim + d] = acc[rr];
+#pragma unroll
+  for (int mp = 0; mp < MAPS; mp++) {
+    float* ow = os + (mp * STK_DW + wave) * vdim;
+    if (vec) {
+      for (int o = oc; o < 64; o <<= 1)
+        for (int i = 0; i < 8; i++) vacc[mp][i] += __shfl_xor(vacc[mp][i], o, 64);
+      if (lane < oc && co * 8 < vdim)
+        for (int i = 0; i < 8; i++) ow[co * 8 + i] = vacc[mp][i];
+    } else {
+      for (int rr = 0; rr < NR; rr++) {
+        const int d = lane + 64 * rr;
+        if (d < vdim) ow[d] = acc[mp][rr];
+      }
     }
+    if (lane == 0) ms[mp * 2 * STK_DW + wave] = m[mp], ms[mp * 2 * STK_DW + STK_DW + wave] = l[mp];
   }
-  if (lane == 0) ms[wave] = m, ms[STK_DW + wave] = l;
   __syncthreads();
-  float M = ms[0];
-  for (int w = 1; w < STK_DW; w++) M = fmaxf(M, ms[w]);
   T* out = (T*)a.out + (size_t)b * a.H * vdim + h * vdim;
   const float og = a.gate ? sigmoidf_(a.gate[(size_t)b * a.gate_ld + h]) : 1.f;
-  for (int d = tid; d < vdim; d += 64 * STK_DW) {
+  auto joined = [&](int mp, int d) {  // the waves' partial sums of channel d, in wave order
+    const float *mm = ms + mp * 2 * STK_DW, *ow = os + mp * STK_DW * vdim;
+    float M = mm[0];
+    for (int w = 1; w < STK_DW; w++) M = fmaxf(M, mm[w]);
     float L = 0.f, o = 0.f;
     for (int w = 0; w < STK_DW; w++) {
-      const float c = ms[w] > -INFINITY ? expf(ms[w] - M) : 0.f;
-      L += ms[STK_DW + w] * c;
-      o += os[w * vdim + d] * c;
+      const float c = mm[w] > -INFINITY ? expf(mm[w] - M) : 0.f;
+      L += mm[STK_DW + w] * c;
+      o += ow[w * vdim + d] * c;
     }
-    El<T>::st(out + d, L > 0.f ? o / L * og : 0.f);
+    return L > 0.f ? o / L : 0.f;
+  };
+  if constexpr (MAPS == 2) {  // (vdim <= 512: a channel a thread)
+    const float o = tid < vdim ? joined(0, tid) - a.diff_lambda * joined(1, tid) : 0.f;
+    const float q2 = wave_sum(o * o);
+    if (lane == 0) qs[wave] = q2;  // (ps and qs are free: every wave has passed the barrier)
+    __syncthreads();
+    float t2 = qs[0];
+    for (int w = 1; w < STK_DW; w++) t2 += qs[w];
+    if (tid < vdim) El<T>::st(out + tid, o * (a.diff_scale / sqrtf(t2 / (float)vdim + a.diff_eps)));
+    return;
   }
+  for (int d = tid; d < vdim; d += 64 * STK_DW) El<T>::st(out + d, joined(0, d) * og);
 }
 
 }  // namespace
@@ -984,7 +1090,7 @@ void vra_stack_gemm(const StkGemmArgs& g, int dtype, int64_t stream) {
   const bool big = g.tile_group ? g.granule == 64 : g.M > 32;
   const bool mfma = dtype == VRA_BF16 && g.K % 8 == 0 && g.lda % 8 == 0 && ((uintptr_t)g.a % 16 == 0) && ((uintptr_t)g.w % 16 == 0) &&
                     (g.w_group_stride % 8 == 0) && (g.a_batch_stride % 8 == 0) && (g.w_batch_stride % 8 == 0);
-  VRA_CHECK_ARG(g.epi >= 0 && g.epi <= 2 && (g.epi != 2 || g.act == 3) && (g.softcap <= 0.f || g.epi != 1), "stack gemm: unknown epilogue");
+  VRA_CHECK_ARG(g.epi >= 0 && g.epi <= 2 && (g.epi != 2 || (g.act >= 3 && g.act <= 6)) && (g.softcap <= 0.f || g.epi != 1), "stack gemm: unknown epilogue");
   const bool post = g.epi == 2 || g.softcap > 0.f;
   VRA_CHECK_ARG(!post || !g.a_scale, "stack gemm: scaled rows and an element-wise epilogue do not come together");
   VRA_CHECK_ARG(g.epi != 1 || (mfma && g.N % 32 == 0), "stack gemm: the gated epilogue needs the bf16 MFMA path and whole gate / up blocks");
@@ -1086,13 +1192,21 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
   VRA_CHECK_ARG(a.q && a.out && a.kc && a.vc && a.positions && a.block_tables && a.context_lens, "stack attention: null pointer");
   VRA_CHECK_ARG(a.B > 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.dim > 0 && a.vdim > 0 && a.vdim <= 512 && a.BS > 0 && a.max_blocks > 0,
                 "stack attention: heads must be a multiple of kv heads, value size at most 512");
+  VRA_CHECK_ARG(a.maps == 1 || (a.maps == 2 && !a.sink && !a.gate && !a.head_scale && a.chunk <= 0 && a.window <= 0 && a.softcap <= 0.f && a.temp_every <= 0),
+                "stack attention: the differential form has two maps and no sink, gate, head scale, mask, cap or temperature");
+  const bool two = a.maps == 2;
+  const size_t dm = (size_t)a.maps * a.dim;
   hipStream_t st = as_stream(stream);
   if (!a.cu_q) {
-    if (vra_stack_latent_decode(a, dtype, stream)) return;
-    const size_t lds = ((size_t)a.dim + 2 * STK_DW * 64 + 2 * STK_DW + STK_DW * (size_t)a.vdim) * sizeof(float);
+    if (!two && vra_stack_latent_decode(a, dtype, stream)) return;
+    const size_t lds = (std::max<size_t>(dm, STK_DW) + (a.maps + 1) * STK_DW * 64 + a.maps * (2 * STK_DW + STK_DW * (size_t)a.vdim)) * sizeof(float);
     VRA_CHECK_ARG(lds <= 64 * 1024, "stack attention: head does not fit LDS");
     dim3 grid(a.B, a.H);
-#define STK_DEC(TT, NRV) launch_checked("stack attention (decode)", [&] { stk_attn_decode_kernel<TT, NRV><<<grid, 64 * STK_DW, lds, st>>>(a); })
+#define STK_DEC(TT, NRV)                                                                              \
+  launch_checked("stack attention (decode)", [&] {                                                    \
+    if (two) stk_attn_decode_kernel<TT, NRV, 2><<<grid, 64 * STK_DW, lds, st>>>(a);                   \
+    else stk_attn_decode_kernel<TT, NRV, 1><<<grid, 64 * STK_DW, lds, st>>>(a);                       \
+  })
     if (dtype == VRA_F32) {
       if (a.vdim <= 256) STK_DEC(float, 4);
       else STK_DEC(float, 8);
@@ -1103,27 +1217,40 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
 #undef STK_DEC
     return;
   }
-  if (vra_stack_latent_prefill(a, dtype, stream)) return;
+  if (!two && vra_stack_latent_prefill(a, dtype, stream)) return;
   if (dtype == VRA_BF16 && a.dim % 8 == 0 && a.vdim % 16 == 0 && a.dim <= 256 && a.vdim <= 256 && a.ldq % 8 == 0 && ((uintptr_t)a.q % 16 == 0) && a.BS % 32 == 0 &&
       a.k_ld % 8 == 0 && a.v_ld % 8 == 0 && ((uintptr_t)a.vc % 16 == 0)) {
     dim3 grid((a.max_q + 63) / 64, a.B, a.H);
-#define STK_PFM(DCV, VTV) launch_checked("stack attention (prefill, mfma)", [&] { stk_attn_prefill_mfma_kernel<DCV, VTV><<<grid, 256, 0, st>>>(a); })
-    if (a.dim <= 64 && a.vdim <= 64) STK_PFM(2, 4);
+#define STK_PFMN(DCV, VTV, MV) launch_checked("stack attention (prefill, mfma)", [&] { stk_attn_prefill_mfma_kernel<DCV, VTV, MV><<<grid, 256 * MV, 0, st>>>(a); })
+#define STK_PFM(DCV, VTV) STK_PFMN(DCV, VTV, 1)
+    if (two) {
+      if (a.dim <= 64 && a.vdim <= 64) STK_PFMN(2, 4, 2);
+      else if (a.dim <= 64 && a.vdim <= 128) STK_PFMN(2, 8, 2);
+      else if (a.dim <= 128 && a.vdim <= 128) STK_PFMN(4, 8, 2);
+      else if (a.dim <= 128) STK_PFMN(4, 16, 2);
+      else STK_PFMN(8, 16, 2);
+    } else if (a.dim <= 64 && a.vdim <= 64) STK_PFM(2, 4);
     else if (a.dim <= 128 && a.vdim <= 128) STK_PFM(4, 8);
     else if (a.vdim <= 192) STK_PFM(8, 12);  // (a latent cache's rows: 192 value channels do not pay for 256)
     else STK_PFM(8, 16);
 #undef STK_PFM
+#undef STK_PFMN
     return;
   }
-  auto need = [&](int kt) { return ((size_t)STK_QT * a.dim + (size_t)kt * (a.dim + 1) + (size_t)kt * a.vdim + (size_t)STK_QT * kt) * sizeof(float); };
+  auto need = [&](int kt) { return ((size_t)STK_QT * dm + (size_t)kt * (dm + 1) + (size_t)kt * a.vdim + (size_t)a.maps * STK_QT * kt) * sizeof(float); };
   dim3 grid((a.max_q + STK_QT - 1) / STK_QT, a.B, a.H);
   const int kt = need(64) <= 64 * 1024 ? 64 : (need(32) <= 64 * 1024 ? 32 : 16);
   const size_t lds = need(kt);
   VRA_CHECK_ARG(lds <= 160 * 1024, "stack attention: head does not fit LDS");
-#define STK_PFN(TT, KTV, NRV)                                                                                                                     \
+#define STK_PFM2(TT, KTV, NRV, MV)                                                                                                                \
   do {                                                                                                                                            \
-    if (lds > 64 * 1024) (void)hipFuncSetAttribute((const void*)stk_attn_prefill_kernel<TT, KTV, NRV>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
-    launch_checked("stack attention (prefill)", [&] { stk_attn_prefill_kernel<TT, KTV, NRV><<<grid, 256, lds, st>>>(a); });                         \
+    if (lds > 64 * 1024) (void)hipFuncSetAttribute((const void*)stk_attn_prefill_kernel<TT, KTV, NRV, MV>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+    launch_checked("stack attention (prefill)", [&] { stk_attn_prefill_kernel<TT, KTV, NRV, MV><<<grid, 256, lds, st>>>(a); });                     \
+  } while (0)
+#define STK_PFN(TT, KTV, NRV)              \
+  do {                                     \
+    if (two) STK_PFM2(TT, KTV, NRV, 2);    \
+    else STK_PFM2(TT, KTV, NRV, 1);        \
   } while (0)
 #define STK_PF(TT, KTV)                      \
   do {                                       \
@@ -1141,6 +1268,7 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
   }
 #undef STK_PF
 #undef STK_PFN
+#undef STK_PFM2
 }
 
 // ================================================================================================ C entry points (one operator each)

@@ -197,9 +197,9 @@ __device__ void router_pick(const StkSandwichArgs& a, int t, float* zs) {
     const float norm = sig ? sum + 1e-20f : 1.f;
     if (lane < a.top) {
       a.pair_expert[(size_t)t * a.top + lane] = pick_e;
-      a.pair_weight[(size_t)t * a.top + lane] = sig ? pick_w / norm : pick_w;
+      a.pair_weight[(size_t)t * a.top + lane] = sig ? pick_w / norm : pick_w * a.weight_scale;
     }
-    if (lane == 0 && a.id_weight) a.id_weight[t] = idw / norm;
+    if (lane == 0 && a.id_weight) a.id_weight[t] = sig ? idw / norm : idw * a.weight_scale;
     return;
   }
   if (tid != 0) return;
@@ -213,13 +213,13 @@ __device__ void router_pick(const StkSandwichArgs& a, int t, float* zs) {
     sc[best] = -1.f;  // (picked: out of the list)
     const bool ident = best >= n_real;
     a.pair_expert[(size_t)t * a.top + j] = ident ? -1 : best;
-    a.pair_weight[(size_t)t * a.top + j] = w;
+    a.pair_weight[(size_t)t * a.top + j] = sig ? w : w * a.weight_scale;
     if (ident) idw += w;
     sum += w;
   }
   if (sig)
     for (int j = 0; j < a.top; j++) a.pair_weight[(size_t)t * a.top + j] /= sum + 1e-20f;
-  if (a.id_weight) a.id_weight[t] = sig ? idw / (sum + 1e-20f) : idw;
+  if (a.id_weight) a.id_weight[t] = sig ? idw / (sum + 1e-20f) : idw * a.weight_scale;
 }
 
 // any width
@@ -270,6 +270,7 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
         if (a.p2_norm_w) v2 = v2 * r2 * a.p2_norm_w[c];
         v = fmaf(a.c2 * w2, v2, v);
       }
+      if (a.xw) v = fmaf(a.xw[t], x[c], v);
       xs[c] = v;
       s = fmaf(v, v, s);
     }
@@ -297,9 +298,10 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   } else {
     for (int c = tid; c < W; c += 256) xs[c] = x[c];
   }
-  if (!a.pre_w) return;
+  if (!a.pre_w && !a.pre_identity) return;
   float r = 1.f;
-  if (a.norm_kind == 2) {
+  if (a.pre_identity) {
+  } else if (a.norm_kind == 2) {
     r = center_rows(xs, W, tid, a.eps, red);
   } else if (a.norm_kind == 0) {
     float s = 0.f;
@@ -308,7 +310,7 @@ __global__ __launch_bounds__(256) void stk_sandwich_kernel(StkSandwichArgs a) {
   }
   T* h = (T*)a.h + (size_t)t * W;
   for (int c = tid; c < W; c += 256) {
-    const float v = a.norm_kind == 1 ? tanhf(a.pre_alpha * xs[c]) * a.pre_w[c] + a.pre_b[c] : xs[c] * r * a.pre_w[c];
+    const float v = a.pre_identity ? xs[c] : (a.norm_kind == 1 ? tanhf(a.pre_alpha * xs[c]) * a.pre_w[c] + a.pre_b[c] : xs[c] * r * a.pre_w[c]);
     xs[c] = v;
     El<T>::st(h + c, v);
     if (a.h32) a.h32[(size_t)t * W + c] = v;
@@ -418,7 +420,7 @@ __global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
       p2[v] = ld4(a.p2 ? a.p2 + (size_t)t * W + col[v] : x, in[v] && a.p2);
       s[v] = make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    const float w2 = a.c2 * (a.p2w ? a.p2w[t] : 1.f);
+    const float w2 = a.c2 * (a.p2w ? a.p2w[t] : 1.f), wx = a.xw ? a.xw[t] : 0.f;
     if (a.n1 == 1 && !a.pw && !a.pe) {
 #pragma unroll
       for (int v = 0; v < NV; v++) s[v] = ld4(a.p1 + (size_t)t * W + col[v], in[v]);
@@ -463,6 +465,7 @@ __global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
     for (int v = 0; v < NV; v++) {
       s[v].x = fmaf(w2, p2[v].x, s[v].x * a.c1), s[v].y = fmaf(w2, p2[v].y, s[v].y * a.c1);
       s[v].z = fmaf(w2, p2[v].z, s[v].z * a.c1), s[v].w = fmaf(w2, p2[v].w, s[v].w * a.c1);
+      if (a.xw) s[v].x = fmaf(wx, xv[v].x, s[v].x), s[v].y = fmaf(wx, xv[v].y, s[v].y), s[v].z = fmaf(wx, xv[v].z, s[v].z), s[v].w = fmaf(wx, xv[v].w, s[v].w);
     }
     if (a.norm_kind == 1) {
 #pragma unroll
@@ -497,9 +500,9 @@ __global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
   } else if (PREF && a.router_w && vec8) {
     request_router(wave * EB);
   }
-  if (!a.pre_w) return;
+  if (!a.pre_w && !a.pre_identity) return;
   float r = 1.f;
-  if (a.norm_kind == 2) {
+  if (a.norm_kind == 2 && !a.pre_identity) {
     float q = 0.f;
 #pragma unroll
     for (int v = 0; v < NV; v++) q += (xv[v].x + xv[v].y) + (xv[v].z + xv[v].w);
@@ -508,7 +511,7 @@ __global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
     for (int v = 0; v < NV; v++)
       if (in[v]) xv[v].x -= mean, xv[v].y -= mean, xv[v].z -= mean, xv[v].w -= mean;
   }
-  if (a.norm_kind != 1) {
+  if (a.norm_kind != 1 && !a.pre_identity) {
     float q = 0.f;
 #pragma unroll
     for (int v = 0; v < NV; v++) q = dot4(xv[v], q);
@@ -518,9 +521,11 @@ __global__ __launch_bounds__(NT) void stk_seam_vec_kernel(StkSandwichArgs a) {
 #pragma unroll
   for (int v = 0; v < NV; v++) {
     if (!in[v]) continue;
-    const float4 g = *(const float4*)(a.pre_w + col[v]);
+    const float4 g = ld4(a.pre_identity ? x + col[v] : a.pre_w + col[v], !a.pre_identity);
     float4 y;
-    if (a.norm_kind == 1) {
+    if (a.pre_identity) {
+      y = xv[v];
+    } else if (a.norm_kind == 1) {
       const float4 b = *(const float4*)(a.pre_b + col[v]);
       y.x = tanhf(a.pre_alpha * xv[v].x) * g.x + b.x, y.y = tanhf(a.pre_alpha * xv[v].y) * g.y + b.y;
       y.z = tanhf(a.pre_alpha * xv[v].z) * g.z + b.z, y.w = tanhf(a.pre_alpha * xv[v].w) * g.w + b.w;
@@ -729,7 +734,8 @@ __device__ __forceinline__ float group_sum(float v) {
 // P, the presence of per-row decays and of the delta rule are template parameters: the 16 tokens of a tile are one straight line of code, so
 // the LDS reads of the tokens ahead are in flight while a token's sums run.
 // DECAY 0: one constant per head; 1: one per row and key channel; 2: one per row and head.  ACT: q, k, v pass silu on their way into LDS.
-template <int R, int P, int DECAY, bool BETA, bool ACT>
+// BONUS (per-channel decays, no delta rule): the output is read before the decay, this token enters it through bonus (bs: sum_d q_d bonus_d k_d).
+template <int R, int P, int DECAY, bool BETA, bool ACT, bool BONUS = false>
 __global__ __launch_bounds__(256) void stk_linear_scan_kernel(StkScanArgs a) {
   constexpr int TT = 16, NL = 4;     // tokens a tile; 16-byte loads a thread and array for one tile (TT * dimP / 4 / 256, dimP <= 256)
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -753,6 +759,12 @@ __global__ __launch_bounds__(256) void stk_linear_scan_kernel(StkScanArgs a) {
 #pragma unroll
   for (int j = 0; j < R; j++) S[j] = (!fresh && col && r * R + j < dim) ? sp[j] : 0.f;
   const float hd = a.head_decay ? a.head_decay[h] : 1.f;
+  float4 ub = make_float4(0.f, 0.f, 0.f, 0.f);  // this thread's channels of a staged row (256 is a multiple of d4n: the same ones in every load)
+  if (BONUS) {
+    const float* bp = a.bonus + (size_t)h * dim;
+    const int d = (tid % d4n) * 4;
+    ub.x = d < dim ? bp[d] : 0.f, ub.y = d + 1 < dim ? bp[d + 1] : 0.f, ub.z = d + 2 < dim ? bp[d + 2] : 0.f, ub.w = d + 3 < dim ? bp[d + 3] : 0.f;
+  }
   // rows of dim floats that start on 16 bytes are fetched four floats a load
   const bool vec = dim % 4 == 0 && a.ldk % 4 == 0 && a.ldq % 4 == 0 && (DECAY != 1 || a.ldd % 4 == 0) && ((uintptr_t)a.k % 16) == 0 && ((uintptr_t)a.q % 16) == 0 &&
                    (DECAY != 1 || ((uintptr_t)a.decay % 16) == 0);
@@ -807,6 +819,13 @@ __global__ __launch_bounds__(256) void stk_linear_scan_kernel(StkScanArgs a) {
         *(float4*)(qs + e * 4) = qv;
         if (DECAY == 1) *(float4*)(ds + e * 4) = dn[u];
       }
+      if (BONUS) {  // the d4n neighbouring lanes that hold a token's q and k (zeros beyond its size) sum q . (bonus k)
+        const float4 kk = kn[u], qv = qn[u];
+        float c = fmaf(qv.x * ub.x, kk.x, fmaf(qv.y * ub.y, kk.y, fmaf(qv.z * ub.z, kk.z, qv.w * ub.w * kk.w)));
+#pragma unroll
+        for (int o = 1; o < d4n; o <<= 1) c += __shfl_xor(c, o, 64);
+        if (e < TT * d4n && e % d4n == 0) bs[e / d4n] = c * a.q_scale;
+      }
     }
 #pragma unroll
     for (int u = 0; u < 16; u++) {
@@ -837,10 +856,22 @@ __global__ __launch_bounds__(256) void stk_linear_scan_kernel(StkScanArgs a) {
         }
       }
       uv[w] = vs[i * CPB + cl];
-      if (BETA) bv[w] = bs[i];
+      if (BETA || BONUS) bv[w] = bs[i];
       if (DECAY == 2) gv[w] = gs[i];
     };
     auto token = [&](int i, int w) {
+      if (BONUS) {
+        const float u = uv[w];
+        float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+        for (int j = 0; j < R; j += 2) {
+          o0 = fmaf(S[j], qv[w][j], o0), o1 = fmaf(S[j + 1], qv[w][j + 1], o1);
+          S[j] = fmaf(kv[w][j], u, S[j] * dv[w][j]), S[j + 1] = fmaf(kv[w][j + 1], u, S[j + 1] * dv[w][j + 1]);
+        }
+        const float o_ = fmaf(bv[w], u, group_sum<P>(o0 + o1));
+        if (r == 0 && col) a.out[(size_t)(t0 + i0 + i) * a.ldo + h * vdim + c] = o_;
+        return;
+      }
 #pragma unroll
       for (int j = 0; j < R; j++) S[j] *= DECAY == 1 ? dv[w][j] : (DECAY == 2 ? gv[w] : hd);
       float u = uv[w];
@@ -882,7 +913,7 @@ __global__ __launch_bounds__(256) void stk_linear_scan_kernel(StkScanArgs a) {
 // ------------------------------------------------------------------------------------------------ per-head output norm and gate
 template <typename T>
 __global__ __launch_bounds__(256) void stk_head_norm_gate_kernel(const float* o, const float* w, const float* gate, int gate_ld, int gate_act, float eps,
-                                                                 T* out, int H, int vdim) {
+                                                                 T* out, int H, int vdim, int w_per_head) {
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   if (H == 1) {  // one norm over the whole row: the four waves share it
     __shared__ float red[4];
@@ -908,7 +939,7 @@ __global__ __launch_bounds__(256) void stk_head_norm_gate_kernel(const float* o,
     const float r = 1.f / sqrtf(wave_sum(s) / (float)vdim + eps);
     for (int c = lane; c < vdim; c += 64) {
       float v = src[c] * r;
-      if (w) v *= w[c];
+      if (w) v *= w[w_per_head ? h * vdim + c : c];
       if (gate) {
         const float g = gate[(size_t)t * gate_ld + h * vdim + c];
         v *= gate_act == 1 ? siluf_(g) : sigmoidf_(g);
@@ -956,6 +987,53 @@ __global__ __launch_bounds__(256) void stk_conv_rows_update_kernel(StkConvArgs a
       else if (!fresh) v = cs[(size_t)(taps - 1 + e) * C + c];
       cs[(size_t)r * C + c] = v;
     }
+}
+
+// ------------------------------------------------------------------------------------------------ token shift
+// A thread holds V channels of its token's row and of the row before it for all mixes.  The state a sequence's first row reads is written by the
+// same thread (with the sequence's last row, which lies in x), so one launch reads and moves it.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void stk_token_shift_kernel(StkShiftArgs a) {
+  const int t = blockIdx.x, W = a.W, b = seq_of_row(a.cu_q, a.B, t), slot = a.state_slots[b];
+  if (slot < 0) return;
+  const int t0 = a.cu_q ? (int)a.cu_q[b] : t, t1 = a.cu_q ? (int)a.cu_q[b + 1] : t + 1;
+  const bool fresh = a.positions[t0] == 0;
+  T* out = (T*)a.out;
+  for (int c = (blockIdx.y * 256 + threadIdx.x) * V; c < W; c += 256 * V * gridDim.y) {
+    float x[V], d[V];
+    const float* src = a.x + (size_t)t * W + c;
+    float* st = a.shift_state + (size_t)slot * W + c;
+    const float* pre = t > t0 ? src - W : st;
+    if constexpr (V == 4) {
+      const float4 xv = *(const float4*)src, pv = *(const float4*)pre;
+      x[0] = xv.x, x[1] = xv.y, x[2] = xv.z, x[3] = xv.w, d[0] = pv.x, d[1] = pv.y, d[2] = pv.z, d[3] = pv.w;
+    } else {
+      x[0] = *src, d[0] = *pre;
+    }
+#pragma unroll
+    for (int i = 0; i < V; i++) d[i] = (t == t0 && fresh ? 0.f : d[i]) - x[i];
+    if (t == t0) {
+#pragma unroll
+      for (int i = 0; i < V; i++) st[i] = a.x[(size_t)(t1 - 1) * W + c + i];
+    }
+    for (int m = 0; m < a.n; m++) {
+      const float* mu = a.mu + (size_t)m * W + c;
+      T* o = out + ((size_t)m * a.T + t) * W + c;
+      if constexpr (V == 4) {
+        const float4 u = *(const float4*)mu;
+        const float y0 = fmaf(d[0], u.x, x[0]), y1 = fmaf(d[1], u.y, x[1]), y2 = fmaf(d[2], u.z, x[2]), y3 = fmaf(d[3], u.w, x[3]);
+        if constexpr (sizeof(T) == 2) {
+          uint2 p;
+          p.x = BF16::pack2(y0, y1), p.y = BF16::pack2(y2, y3);
+          *(uint2*)o = p;
+        } else {
+          *(float4*)o = make_float4(y0, y1, y2, y3);
+        }
+      } else {
+        El<T>::st(o, fmaf(d[0], mu[0], x[0]));
+      }
+    }
+  }
 }
 
 // ------------------------------------------------------------------------------------------------ real-gated diagonal recurrence
@@ -1054,8 +1132,10 @@ void vra_stack_embed_pair(const StkEmbedPairArgs& a, int dtype, int64_t stream) 
 }
 
 void vra_stack_sandwich_norm(const StkSandwichArgs& a, int dtype, int64_t stream) {
-  VRA_CHECK_ARG(a.x && a.T > 0 && a.W > 0 && (!a.post_w || (a.p1 && a.n1 >= 1)) && (!a.pre_w || a.h), "stack seam norm: null pointer or empty shape");
-  VRA_CHECK_ARG(!a.router_w || (a.pre_w && a.pair_expert && a.pair_weight && a.top >= 1 && a.top <= a.n_router), "stack seam norm: router outputs");
+  VRA_CHECK_ARG(a.x && a.T > 0 && a.W > 0 && (!a.post_w || (a.p1 && a.n1 >= 1)) && (!(a.pre_w || a.pre_identity) || a.h) && !(a.pre_w && a.pre_identity),
+                "stack seam norm: null pointer or empty shape");
+  VRA_CHECK_ARG(!a.router_w || ((a.pre_w || a.pre_identity) && a.pair_expert && a.pair_weight && a.top >= 1 && a.top <= a.n_router),
+                "stack seam norm: router outputs");
   VRA_CHECK_ARG(a.norm_kind >= 0 && a.norm_kind <= 2 && a.router_kind >= 0 && a.router_kind <= 2, "stack seam norm: unknown norm or router kind");
   VRA_CHECK_ARG(a.norm_kind != 1 || ((!a.post_w || a.post_b) && (!a.pre_w || a.pre_b)), "stack seam norm: Dynamic Tanh needs its offsets");
   VRA_CHECK_ARG((!a.p1_norm_w && !a.p2_norm_w) || a.n1 == 1, "stack seam norm: a part with a norm of its own is one row a token");
@@ -1137,10 +1217,12 @@ void vra_stack_linear_scan(const StkScanArgs& a, int64_t stream) {
   const bool decay = a.decay != nullptr, beta = a.beta != nullptr, per_head = decay && a.decay_per_head;
   VRA_CHECK_ARG(decay || !beta, "stack linear scan: the delta rule comes with per-row decays");
   VRA_CHECK_ARG(!a.act_silu || (!decay && !beta), "stack linear scan: the activation on the way in goes with constant decays");
+  VRA_CHECK_ARG(!a.bonus || (decay && !per_head && !beta), "stack linear scan: the bonus goes with per-row decays per channel, without the delta rule");
   VRA_CHECK_ARG(!per_head || beta, "stack linear scan: one decay per head and token goes with the delta rule");
 #define STK_SCAN(PV)                                                                                                            \
   launch_checked("stack linear scan", [&] {                                                                                     \
-    if (per_head) stk_linear_scan_kernel<R, PV, 2, true, false><<<grid, 256, lds, st>>>(a);                                     \
+    if (a.bonus) stk_linear_scan_kernel<R, PV, 1, false, false, true><<<grid, 256, lds, st>>>(a);                               \
+    else if (per_head) stk_linear_scan_kernel<R, PV, 2, true, false><<<grid, 256, lds, st>>>(a);                                \
     else if (beta) stk_linear_scan_kernel<R, PV, 1, true, false><<<grid, 256, lds, st>>>(a);                                    \
     else if (decay) stk_linear_scan_kernel<R, PV, 1, false, false><<<grid, 256, lds, st>>>(a);                                  \
     else if (a.act_silu) stk_linear_scan_kernel<R, PV, 0, false, true><<<grid, 256, lds, st>>>(a);                              \
@@ -1158,13 +1240,13 @@ void vra_stack_linear_scan(const StkScanArgs& a, int64_t stream) {
 }
 
 void vra_stack_head_norm_gate(const float* o, const float* w, const float* gate, int gate_ld, int gate_act, float eps, void* out, int T, int H, int vdim,
-                              int dtype, int64_t stream) {
+                              int dtype, int64_t stream, int w_per_head) {
   VRA_CHECK_ARG(o && out && T > 0 && H > 0 && vdim > 0, "stack head norm: null pointer or empty shape");
   if (dtype == VRA_F32)
-    launch_checked("stack head norm", [&] { stk_head_norm_gate_kernel<float><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (float*)out, H, vdim); });
+    launch_checked("stack head norm", [&] { stk_head_norm_gate_kernel<float><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (float*)out, H, vdim, w_per_head); });
   else
     launch_checked("stack head norm", [&] {
-      stk_head_norm_gate_kernel<uint16_t><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (uint16_t*)out, H, vdim);
+      stk_head_norm_gate_kernel<uint16_t><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (uint16_t*)out, H, vdim, w_per_head);
     });
 }
 
@@ -1182,6 +1264,20 @@ void vra_stack_conv_rows_update(const StkConvArgs& a, int64_t stream) {
   VRA_CHECK_ARG(a.conv_state, "stack convolution state: null pointer");
   const dim3 grid(a.B, std::min((a.C + 255) / 256, 64));
   launch_checked("stack convolution state", [&] { stk_conv_rows_update_kernel<<<grid, 256, 0, as_stream(stream)>>>(a); });
+}
+void vra_stack_token_shift(const StkShiftArgs& a, int dtype, int64_t stream) {
+  VRA_CHECK_ARG(a.x && a.mu && a.shift_state && a.positions && a.state_slots && a.out, "stack token shift: null pointer");
+  VRA_CHECK_ARG(a.T > 0 && a.B > 0 && a.W > 0 && a.n > 0 && (a.cu_q || a.T == a.B), "stack token shift: shapes");
+  auto al16 = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  const bool v4 = a.W % 4 == 0 && al16(a.x) && al16(a.mu) && al16(a.shift_state) && al16(a.out);
+  const dim3 grid(a.T, std::min((a.W + 1023) / 1024, 64));
+  hipStream_t st = as_stream(stream);
+  launch_checked("stack token shift", [&] {
+    if (dtype == VRA_F32 && v4) stk_token_shift_kernel<float, 4><<<grid, 256, 0, st>>>(a);
+    else if (dtype == VRA_F32) stk_token_shift_kernel<float, 1><<<grid, 256, 0, st>>>(a);
+    else if (v4) stk_token_shift_kernel<uint16_t, 4><<<grid, 256, 0, st>>>(a);
+    else stk_token_shift_kernel<uint16_t, 1><<<grid, 256, 0, st>>>(a);
+  });
 }
 void vra_stack_gated_scan(const StkGatedScanArgs& a, int T, int dtype, int64_t stream) {
   VRA_CHECK_ARG(a.u && a.gr && a.gi && a.y && a.lam && a.state && a.state_slots && a.positions && a.out, "stack gated scan: null pointer");

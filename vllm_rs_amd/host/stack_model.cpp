@@ -60,13 +60,14 @@ bool StackModel::parse_spec(const char* spec) {
       width_ = (int)num("width", 0), vocab_ = (int)num("vocab", 0), groups_ = (int)num("groups", 1);
       eps_ = (float)num("eps", 1e-6), residual_mult_ = (float)num("residual_mult", 1.0), logit_scale_ = (float)num("logit_scale", 1.0);
       pos_base_ = num("pos_base", 10000.0);
-      auto pick = [&](const char* k, const char* a, const char* b, int* out, const char* c = nullptr) {
+      auto pick = [&](const char* k, const char* a, const char* b, int* out, const char* c = nullptr, const char* d = nullptr) {
         const std::string v = f.count(k) ? f[k] : a;
-        if (v != a && v != b && !(c && v == c)) return spec_error_ = std::string("layer stack spec: ") + k + " must be " + a + " or " + b + (c ? std::string(" or ") + c : ""), false;
-        *out = v == b ? 1 : (c && v == c ? 2 : 0);
+        if (v != a && v != b && !(c && v == c) && !(d && v == d))
+          return spec_error_ = std::string("layer stack spec: ") + k + " must be " + a + " or " + b + (c ? std::string(" or ") + c : "") + (d ? std::string(" or ") + d : ""), false;
+        *out = v == b ? 1 : (c && v == c ? 2 : (d && v == d ? 3 : 0));
         return true;
       };
-      if (!pick("block", "parallel", "sequential", &block_, "sandwich") || !pick("norm", "rms", "dyt", &norm_kind_, "layer") || !pick("pos", "sinusoid", "none", &pos_kind_))
+      if (!pick("block", "parallel", "sequential", &block_, "sandwich", "post") || !pick("norm", "rms", "dyt", &norm_kind_, "layer") || !pick("pos", "sinusoid", "none", &pos_kind_))
         return false;
       norm_offset_ = (float)num("norm_offset", 0.0), embed_scale_ = (float)num("embed_scale", 1.0), embed_norm_ = (int)num("embed_norm", 0);
       pair_buckets_ = (int)num("pair_buckets", 0), pair_mul_prev_ = (int64_t)num("pair_mul_prev", 0), pair_mul_cur_ = (int64_t)num("pair_mul_cur", 0);
@@ -77,10 +78,13 @@ bool StackModel::parse_spec(const char* spec) {
       L.scale = (float)num("scale", L.dim > 0 ? 1.0 / sqrt((double)L.dim) : 1.0), L.softcap = (float)num("softcap", 0.0);
       L.temp_coef = (float)num("temp_coef", 0.0), L.temp_every = (int)num("temp_every", 0), L.kv_from = (int)num("kv_from", -1);
       const std::string mix = f.count("mixer") ? f["mixer"] : "attention";
-      L.mixer = mix == "latent" ? 1 : (mix == "sigmoid" ? 2 : (mix == "delta" ? 3 : (mix == "retention" ? 4 : (mix == "parallel" ? 5 : (mix == "lightning" ? 6 : 0)))));
+      L.mixer = mix == "latent" ? 1 : (mix == "sigmoid" ? 2 : (mix == "delta" ? 3 : (mix == "retention" ? 4 : (mix == "parallel" ? 5 : (mix == "lightning" ? 6 : (mix == "differential" ? 7 : (mix == "wkv" ? 8 : 0)))))));
       if (mix != "attention" && L.mixer == 0) return spec_error_ = "layer stack spec: unknown mixer " + mix, false;
+      if (L.mixer == 7) L.maps = 2, L.diff = (float)num("diff", 0.0), L.qk_norm = 1, L.has_bias = 1;
+      L.router_scale = (float)num("router_scale", 1.0);
       L.conv = (int)num("conv", 0), L.rank_a = (int)num("rank_a", 0), L.rank_g = (int)num("rank_g", 0), L.chunk = (int)num("chunk", 0);
       L.qk_norm = (int)num("qk_norm", 0), L.has_bias = (int)num("bias", 0);
+      if (L.mixer == 8) L.conv = 2, L.shift_w = width_;  // (the previous token's row is carried like the one earlier input of a two-tap convolution)
       L.rs_factor = num("rs_factor", 0.0), L.rs_low = num("rs_low", 1.0), L.rs_high = num("rs_high", 4.0), L.rs_original = num("rs_original", 0.0);
       L.r_heads = (int)num("r_heads", 0), L.r_dim = (int)num("r_dim", 0), L.r_vdim = (int)num("r_vdim", L.r_dim), L.tau = (float)num("tau", 1.0);
       L.left_scale = (float)num("left_scale", 1.0), L.right_scale = (float)num("right_scale", 1.0);
@@ -110,8 +114,8 @@ bool StackModel::parse_spec(const char* spec) {
       L.yarn_original = num("yarn_original", 0.0), L.yarn_fast = num("yarn_fast", 32.0), L.yarn_slow = num("yarn_slow", 1.0);
       L.window = (int)num("window", 0), L.keep_first = (int)num("keep_first", 0), L.slope_exp = num("slope_exp", 0.0);
       const std::string mlp = f.count("mlp") ? f["mlp"] : "none";
-      L.mlp = mlp == "dense" ? 1 : (mlp == "moe" ? 2 : (mlp == "gated" ? 3 : (mlp == "clamped" ? 4 : 0)));
-      if (mlp != "dense" && mlp != "moe" && mlp != "none" && mlp != "gated" && mlp != "clamped") return spec_error_ = "layer stack spec: unknown feed-forward kind " + mlp, false;
+      L.mlp = mlp == "dense" ? 1 : (mlp == "moe" ? 2 : (mlp == "gated" ? 3 : (mlp == "clamped" ? 4 : (mlp == "relu2" ? 5 : 0))));
+      if (mlp != "dense" && mlp != "moe" && mlp != "none" && mlp != "gated" && mlp != "clamped" && mlp != "relu2") return spec_error_ = "layer stack spec: unknown feed-forward kind " + mlp, false;
       L.ff = (int)num("ff", 0), L.experts = (int)num("experts", 0), L.top = (int)num("top", 1), L.limit = (float)num("limit", 0.0);
       L.shared_ff = (int)num("shared_ff", 0), L.shared_limit = (float)num("shared_limit", 0.0);
       layers_.push_back(L);
@@ -121,6 +125,7 @@ bool StackModel::parse_spec(const char* spec) {
   }
   if (!have_stack || width_ <= 0 || vocab_ <= 0 || layers_.empty()) return spec_error_ = "layer stack spec: width, vocab and at least one layer are needed", false;
   if (norm_kind_ == 2 && block_ != 2) return spec_error_ = "layer stack spec: layer norms belong to sandwich blocks", false;
+  if (block_ == 3 && norm_kind_ != 0) return spec_error_ = "layer stack spec: post blocks have rms norms", false;
   if (layer_scale_ && (block_ != 2 || norm_kind_ == 1)) return spec_error_ = "layer stack spec: layer_scale belongs to sandwich blocks with rms or layer norms", false;
   if (groups_ < 1 || width_ % groups_) return spec_error_ = "layer stack spec: the width must split into equal norm groups", false;
   if (width_ != mc_.hidden_size || vocab_ != mc_.vocab_size || (int)layers_.size() != mc_.num_layers)
@@ -133,7 +138,15 @@ bool StackModel::parse_spec(const char* spec) {
     if ((L.mixer == 2 && block_ != 1) || (L.mixer == 1 && block_ == 0))
       return spec_error_ = "layer stack spec: latent and sigmoid mixers run in sequential blocks, the latent one also in sandwich blocks" + at, false;
     if (L.mixer == 0 && block_ != 0) return spec_error_ = "layer stack spec: the softmax mixer with temperature and cap runs in parallel blocks" + at, false;
-    if (L.mixer >= 3 && block_ != 2) return spec_error_ = "layer stack spec: delta, retention and parallel mixers run in sandwich blocks" + at, false;
+    if ((L.mixer >= 7) != (block_ == 3)) return spec_error_ = "layer stack spec: post blocks hold differential and wkv mixers" + at, false;
+    if (L.mixer == 7 && L.vdim > 512) return spec_error_ = "layer stack spec: differential attention takes value sizes up to 512" + at, false;
+    if (L.mixer == 8 && (L.dim > 256 || L.vdim != L.dim || L.kv_heads != L.heads || L.rank_a < 1))
+      return spec_error_ = "layer stack spec: wkv needs dim <= 256, vdim = dim, kv_heads = heads, rank_a" + at, false;
+    if (block_ == 3 && ((L.mlp != 0 && L.mlp != 2 && L.mlp != 5) || L.weights_of >= 0 || (L.mlp == 2 && (L.router_kind != 2 || L.act_kind != 2))))
+      return spec_error_ = "layer stack spec: post blocks have a squared-relu feed-forward, a mixture of experts with router=softmax_all and act=silu, or none, and tensors of their own" + at, false;
+    if (L.mlp == 5 && block_ != 3) return spec_error_ = "layer stack spec: the squared-relu feed-forward belongs to post blocks" + at, false;
+    if (L.router_scale != 1.f && L.router_kind != 2) return spec_error_ = "layer stack spec: router_scale belongs to router=softmax_all" + at, false;
+    if (L.mixer >= 3 && L.mixer < 7 && block_ != 2) return spec_error_ = "layer stack spec: delta, retention and parallel mixers run in sandwich blocks" + at, false;
     if (block_ == 2 && ((L.mixer < 3 && L.mixer != 1) || (L.mlp != 0 && L.mlp != 2 && L.mlp != 4)))
       return spec_error_ = "layer stack spec: sandwich blocks hold latent, delta, retention, lightning or parallel mixers and a mixture of experts, a clamped dense feed-forward or none" + at, false;
     if (block_ == 2 && L.weights_of >= 0 && L.mixer != 1) return spec_error_ = "layer stack spec: in sandwich blocks only layers with the latent mixer share weights" + at, false;
@@ -158,8 +171,8 @@ bool StackModel::parse_spec(const char* spec) {
                          L.chunk < 0 || L.vdim > 256 || (L.rs_factor > 0.0 && (L.rs_original <= 0.0 || L.rs_high <= L.rs_low))))
       return spec_error_ = "layer stack spec: the parallel mixer needs r_heads, r_dim <= 256, r_vdim, rank_a, tau > 0, an even rot_dims <= dim, vdim <= 256" + at, false;
     if (L.router_kind == 3 && block_ != 2) return spec_error_ = "layer stack spec: the normalised sigmoid router belongs to sandwich blocks" + at, false;
-    if ((L.router_kind == 1 || L.router_kind == 2) && (block_ != 2 || L.shared_ff > 0)) return spec_error_ = "layer stack spec: the softmax router belongs to sandwich blocks and has no shared expert" + at, false;
-    if (L.mixer != 0 && L.kv_from >= 0) return spec_error_ = "layer stack spec: kv_from belongs to the softmax mixer" + at, false;
+    if ((L.router_kind == 1 || L.router_kind == 2) && !(block_ == 3 && L.router_kind == 2) && (block_ != 2 || L.shared_ff > 0)) return spec_error_ = "layer stack spec: the softmax router belongs to sandwich blocks and has no shared expert" + at, false;
+    if (L.mixer != 0 && L.mixer != 7 && L.kv_from >= 0) return spec_error_ = "layer stack spec: kv_from belongs to the softmax mixer" + at, false;
     if (L.mixer == 1 && (L.kv_rank <= 0 || L.q_rank <= 0 || L.rot_dim < 0 || L.kv_rank > 512 || L.rot_dims < 0 || L.rot_dims > L.rot_dim || L.rot_dims % 2 ||
                          (L.yarn_factor > 0.0 && (L.yarn_original <= 0.0 || L.yarn_fast <= 0.0 || L.yarn_slow <= 0.0))))
       return spec_error_ = "layer stack spec: latent attention needs q_rank, 0 < kv_rank <= 512, an even rot_dims <= rot_dim" + at, false;
@@ -180,7 +193,7 @@ bool StackModel::parse_spec(const char* spec) {
     } else if (L.kv_from >= 0) {
       if (L.kv_from >= (int)i) return spec_error_ = "layer stack spec: kv_from must name an earlier layer" + at, false;
       const StackLayer& S = layers_[L.kv_from];
-      if (!S.owns_cache || S.kv_heads != L.kv_heads || S.dim != L.dim || S.vdim != L.vdim)
+      if (!S.owns_cache || S.mixer != L.mixer || S.kv_heads != L.kv_heads || S.dim != L.dim || S.vdim != L.vdim)
         return spec_error_ = "layer stack spec: kv_from must name a layer with projections of its own and equal key / value shapes" + at, false;
       L.cache = S.cache;
     } else {
@@ -193,7 +206,7 @@ bool StackModel::parse_spec(const char* spec) {
     if (L.mlp == 2 && (L.ff <= 0 || L.experts <= 0 || L.top < 1 || L.top > L.experts + L.n_identity))
       return spec_error_ = "layer stack spec: mixture of experts needs ff, experts and 1 <= top <= experts" + at, false;
     if (L.mlp == 4 && L.ff <= 0) return spec_error_ = "layer stack spec: clamped feed-forward without ff" + at, false;
-    if (L.mlp == 3 || L.mlp == 4) {
+    if (L.mlp == 3 || L.mlp == 4 || L.mlp == 5) {
       if (L.ff <= 0) return spec_error_ = "layer stack spec: gated feed-forward without ff" + at, false;
       L.shared_ff = L.ff;  // (laid out like a shared expert: gate / up rows interleaved, one weight set for all rows)
     }
@@ -367,7 +380,7 @@ bool StackModel::finalize_weights() {
   else if (!up_mat("head", vocab_, W, &head_)) return false;
   if (block_ == 2 && norm_kind_ == 1) {
     if (!up_norm("final.norm", &final_norm_, &final_b_, &final_alpha_)) return false;
-  } else if (block_ == 2) {
+  } else if (block_ >= 2) {
     if (!up_norm_off("final.norm", W, &final_norm_)) return false;
     if (embed_norm_ && !up_norm_off("embed.norm", W, &embed_norm_w_)) return false;
     if (pair_buckets_ > 0 && !up_mat("bigram", (int64_t)pair_buckets_ + 1, W, &pair_table_)) return false;
@@ -384,6 +397,8 @@ bool StackModel::finalize_weights() {
     } else if (block_ == 2) {
       if (!up_norm_off(p + "norm1", W, &L.norm_w) || !up_norm_scaled(p + "norm1b", p + "ls1", &L.post1_w)) return false;
       if (L.mlp != 0 && (!up_norm_off(p + "norm2", W, &L.norm2_w) || !up_norm_scaled(p + "norm2b", p + "ls2", &L.post2_w))) return false;
+    } else if (block_ == 3) {
+      if (!up_norm_off(p + "norm1", W, &L.post1_w) || (L.mlp != 0 && !up_norm_off(p + "norm2", W, &L.post2_w))) return false;
     } else {
       if (!up_norm(p + "norm1", &L.norm_w, &L.norm_b, &L.norm_alpha)) return false;
       if (block_ == 1 && L.mlp != 0 && !up_norm(p + "norm2", &L.norm2_w, &L.norm2_b, &L.norm2_alpha)) return false;
@@ -420,6 +435,45 @@ bool StackModel::finalize_weights() {
       for (float& r : rate) r = expf(r);
       if (!(L.rate = upload_floats(rate)) || !up_vec(p + "mix.dt_bias", H, &L.dt_bias) || !up_vec(p + "mix.norm", L.vdim, &L.out_norm_w)) return false;
       if (!up_mat(p + "mix.o", W, nv, &L.o)) return false;
+    } else if (L.mixer == 7) {
+      // q (| k | v) in one matrix with one bias row; lambda from its four vectors in f64
+      const HostTensor *q, *k = nullptr, *v = nullptr, *qb, *kb, *vb, *l[4];
+      if (!need(p + "mix.q", L.nq(), W, &q) || !matrix(q) || !need(p + "mix.q.b", L.nq(), -1, &qb)) return false;
+      if (L.owns_cache && (!need(p + "mix.k", L.nk(), W, &k) || !need(p + "mix.v", L.nv(), W, &v) || !matrix(k) || !matrix(v) || !need(p + "mix.k.b", L.nk(), -1, &kb) ||
+                           !need(p + "mix.v.b", L.nv(), -1, &vb) || !up_vec(p + "mix.k.norm", L.dim, &L.kn_w)))
+        return false;
+      std::vector<float> bias;
+      f32_of(*qb, &bias);
+      if (k) f32_of(*kb, &bias), f32_of(*vb, &bias);
+      if (!up_rows(k ? std::vector<const HostTensor*>{q, k, v} : std::vector<const HostTensor*>{q}, &L.qkv) || !(L.qkv_bias = upload_floats(bias))) return false;
+      if (!up_vec(p + "mix.q.norm", L.dim, &L.qn_w) || !up_mat(p + "mix.o", W, L.heads * L.vdim, &L.o) || !up_vec(p + "mix.o.b", W, &L.o_bias)) return false;
+      const char* names[4] = {"mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"};
+      std::vector<float> f[4];
+      for (int i = 0; i < 4; i++) {
+        if (!need(p + names[i], L.dim, -1, &l[i])) return false;
+        f32_of(*l[i], &f[i]);
+      }
+      double s1 = 0.0, s2 = 0.0;
+      for (int i = 0; i < L.dim; i++) s1 += (double)f[0][i] * f[1][i], s2 += (double)f[2][i] * f[3][i];
+      L.lambda = (float)(exp(s1) - exp(s2) + (double)L.diff);
+    } else if (L.mixer == 8) {
+      // r | k | v | gate under one another (each reads a mix of its own: four products of one launch), the decay's low-rank stages apart
+      const int n = L.heads * L.dim;
+      const int64_t ra = rows_of(p + "mix.w1", W);
+      if (ra < 1) return error = "tensor " + p + "mix.w1: missing or of another width", false;
+      L.rank_a = (int)ra;
+      const HostTensor *r, *k, *v, *g, *mu;
+      if (!need(p + "mix.r", n, W, &r) || !need(p + "mix.k", n, W, &k) || !need(p + "mix.v", n, W, &v) || !need(p + "mix.g", n, W, &g) || !matrix(r) || !matrix(k) ||
+          !matrix(v) || !matrix(g) || !up_rows({r, k, v, g}, &L.qkv))
+        return false;
+      std::vector<float> mus;
+      for (const char* c : {"r", "k", "v", "g", "w"}) {
+        if (!need(p + "mix.mu." + c, W, -1, &mu)) return false;
+        f32_of(*mu, &mus);
+      }
+      if (!(L.mu = upload_floats(mus)) || !up_mat(p + "mix.w1", ra, W, &L.lr1) || !up_mat(p + "mix.w2", n, ra, &L.lr2) || !up_vec(p + "mix.w0", n, &L.lr2_bias) ||
+          !up_vec(p + "mix.u", n, &L.bonus) || !up_vec(p + "mix.norm", n, &L.out_norm_w) || !up_mat(p + "mix.o", W, n, &L.o))
+        return false;
     } else if (L.mixer == 6) {
       const int H = L.heads;
       const HostTensor *q, *k, *v, *g;
@@ -590,6 +644,14 @@ bool StackModel::finalize_weights() {
     if (L.mixer < 3 && !up_mat(p + "mix.o", W, L.heads * L.vdim, &L.o)) return false;
     if (L.mlp == 1) {
       if (!up_mat(p + "mlp.up", L.ff, W, &L.up) || !up_mat(p + "mlp.down", W, L.ff, &L.down) || !up_vec(p + "mlp.act", 4, &L.act)) return false;
+    } else if (L.mlp == 5) {
+      const HostTensor *u, *d;
+      if (!need(p + "mlp.up", L.ff, W, &u) || !need(p + "mlp.down", W, L.ff, &d) || !matrix(u) || !matrix(d)) return false;
+      std::vector<uint8_t> su((size_t)L.sffp * W * es, 0), sdn((size_t)W * L.sffp * es);  // (rows beyond ff stay zero)
+      memcpy(su.data(), u->data.data(), u->data.size());
+      pad_cols(d, L.ff, L.sffp, sdn.data());
+      weight_bytes_ += su.size() + sdn.size();
+      if (!(L.s_gu = upload(su.data(), su.size())) || !(L.s_down = upload(sdn.data(), sdn.size()))) return false;
     } else if (L.mlp == 3 || L.mlp == 4) {
       const HostTensor *g, *u, *d;
       if (!need(p + "mlp.gate", L.ff, W, &g) || !need(p + "mlp.up", L.ff, W, &u) || !need(p + "mlp.down", W, L.ff, &d) || !matrix(g) || !matrix(u) || !matrix(d))
@@ -689,7 +751,7 @@ bool StackModel::init_synthetic(uint64_t seed) {
   };
   if (block_ == 2 && norm_kind_ == 1) {
     put_norm("final.norm");
-  } else if (block_ == 2) {  // norm weights are stored around 1 - norm_offset; the embedding's own norm and the token-pair table
+  } else if (block_ >= 2) {  // norm weights are stored around 1 - norm_offset; the embedding's own norm and the token-pair table
     put("final.norm", W, 0, around, 0.05);
     if (embed_norm_) put("embed.norm", W, 0, around, 0.05);
     if (pair_buckets_ > 0) put("bigram", (int64_t)pair_buckets_ + 1, W, 0, 1.0);
@@ -709,6 +771,9 @@ bool StackModel::init_synthetic(uint64_t seed) {
       if (L.mlp != 0) put(p + "norm2", W, 0, around, 0.05), put(p + "norm2b", W, 0, around, 0.05);
       if (layer_scale_) put(p + "ls1", W, 0, 0.8, 0.1);
       if (layer_scale_ && L.mlp != 0) put(p + "ls2", W, 0, 0.8, 0.1);
+    } else if (block_ == 3) {
+      put(p + "norm1", W, 0, around, 0.05);
+      if (L.mlp != 0) put(p + "norm2", W, 0, around, 0.05);
     } else {
       put_norm(p + "norm1");
       if (block_ == 1 && L.mlp != 0) put_norm(p + "norm2");
@@ -720,6 +785,20 @@ bool StackModel::init_synthetic(uint64_t seed) {
       put(p + "mix.a", H, W, 0, sw), put(p + "mix.g", nv, W, 0, sw);
       put(p + "mix.A_log", H, 0, -1.0, 0.5), put(p + "mix.dt_bias", H, 0, -2.0, 1.0), put(p + "mix.norm", L.vdim, 0, 1, 0.05);
       put(p + "mix.o", W, nv, 0, 1.0 / sqrt((double)nv));
+    } else if (L.mixer == 7) {
+      put(p + "mix.q", L.nq(), W, 0, sw), put(p + "mix.q.b", L.nq(), 0, 0, 0.02), put(p + "mix.q.norm", L.dim, 0, 1, 0.05);
+      if (L.owns_cache) {
+        put(p + "mix.k", L.nk(), W, 0, sw), put(p + "mix.k.b", L.nk(), 0, 0, 0.02), put(p + "mix.k.norm", L.dim, 0, 1, 0.05);
+        put(p + "mix.v", L.nv(), W, 0, sw), put(p + "mix.v.b", L.nv(), 0, 0, 0.02);
+      }
+      for (const char* c : {"lq1", "lk1", "lq2", "lk2"}) put(p + "mix." + c, L.dim, 0, 0, 0.1);
+      put(p + "mix.o", W, L.heads * L.vdim, 0, 1.0 / sqrt((double)L.heads * L.vdim)), put(p + "mix.o.b", W, 0, 0, 0.02);
+    } else if (L.mixer == 8) {
+      const int n = L.heads * L.dim;
+      for (const char* c : {"r", "k", "v", "g"}) put(p + "mix." + c, n, W, 0, sw);
+      for (const char* c : {"r", "k", "v", "g", "w"}) put(p + "mix.mu." + c, W, 0, 0.5, 0.2);
+      put(p + "mix.w1", L.rank_a, W, 0, sw), put(p + "mix.w2", n, L.rank_a, 0, 1.0 / sqrt((double)L.rank_a)), put(p + "mix.w0", n, 0, -3.0, 1.0);
+      put(p + "mix.u", L.heads, L.dim, 0.5, 0.3), put(p + "mix.norm", n, 0, 1, 0.05), put(p + "mix.o", W, n, 0, 1.0 / sqrt((double)n));
     } else if (L.mixer == 6) {
       const int H = L.heads;
       put(p + "mix.q", (int64_t)H * L.dim, W, 0, sw), put(p + "mix.k", (int64_t)H * L.dim, W, 0, sw), put(p + "mix.v", (int64_t)H * L.vdim, W, 0, sw);
@@ -784,6 +863,8 @@ bool StackModel::init_synthetic(uint64_t seed) {
     if (L.mixer < 3) put(p + "mix.o", W, L.heads * L.vdim, 0, 1.0 / sqrt((double)L.heads * L.vdim));
     if (L.mlp == 3 || L.mlp == 4) {
       put(p + "mlp.gate", L.ff, W, 0, sw), put(p + "mlp.up", L.ff, W, 0, sw), put(p + "mlp.down", W, L.ff, 0, 1.0 / sqrt((double)L.ff));
+    } else if (L.mlp == 5) {
+      put(p + "mlp.up", L.ff, W, 0, sw), put(p + "mlp.down", W, L.ff, 0, 1.0 / sqrt((double)L.ff));
     } else if (L.mlp == 1) {
       put(p + "mlp.up", L.ff, W, 0, sw), put(p + "mlp.down", W, L.ff, 0, 1.0 / sqrt((double)L.ff));
       HostTensor a;
@@ -906,6 +987,7 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
   size_t nqkv = 0, nattn = 0, zc = 0, actc = 0, top = 0, experts = 0;
   size_t nqa = 0, z2c = 0, recc = 0, roc = 0;
   bool want_h32 = false;
+  size_t nmix = 0;
   for (const StackLayer& L : layers_) {
     // softmax / sigmoid: the joint projection in the model's type; latent: q, later the heads' values (the joint projection is f32 in z_)
     nqkv = std::max(nqkv, L.mixer == 0 ? (size_t)L.nqkv() : std::max((size_t)L.nq(), (size_t)L.heads * L.vdim));
@@ -914,8 +996,9 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
     if (L.mixer == 1) nqa = std::max(nqa, (size_t)L.heads * (L.kv_rank + L.rot_dim)), actc = std::max(actc, T * L.q_rank);
     if (L.mixer != 0) zc = std::max(zc, T * L.nqkv());
     if (L.mlp == 2) top = std::max(top, (size_t)L.top), experts = std::max(experts, (size_t)L.experts);
-    if (L.mlp == 3 || L.mlp == 4) zc = std::max(zc, T * 2 * L.sffp), actc = std::max(actc, T * L.sffp);
+    if (L.mlp == 3 || L.mlp == 4 || L.mlp == 5) zc = std::max(zc, T * 2 * L.sffp), actc = std::max(actc, T * L.sffp);
     if (L.mlp == 2 && L.n_identity > 0) want_h32 = true;
+    if (L.mixer == 8) nmix = 5;
     if (L.mixer == 5 && L.right_kind == 1) {  // the convolved branch in rec_, both gates' logits in z2_, the recurrence's output in attn_
       nattn = std::max(nattn, (size_t)L.r_width), z2c = std::max(z2c, (size_t)2 * L.r_width), recc = std::max(recc, (size_t)L.r_width), roc = std::max<size_t>(roc, 1);
     } else if (L.mixer >= 3) {  // the joint projection is f32 in z_, the low-rank first stages in act_, their second stages in z2_
@@ -923,7 +1006,7 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
       nattn = std::max(nattn, sh * sv);
       actc = std::max(actc, T * (size_t)(L.rank_a + L.rank_g));
       z2c = std::max(z2c, sh * sd + (L.mixer == 3 ? sh * sv : 0));
-      recc = std::max(recc, L.mixer == 3 ? (size_t)L.conv_channels() + sh + sh * sd : (L.mixer == 4 ? 2 * sh * sd : sh * sd));
+      recc = std::max(recc, L.mixer == 3 ? (size_t)L.conv_channels() + sh + sh * sd : (L.mixer == 4 ? 2 * sh * sd : (L.mixer == 8 ? 1 : sh * sd)));
       if (L.mixer == 6) z2c = std::max<size_t>(z2c, 1);
       roc = std::max(roc, sh * sv);
     }
@@ -961,7 +1044,8 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
     lat_scratch_bytes_ = std::max(lat_scratch_bytes_, (size_t)max_seqs * s * L.heads * (L.kv_rank + 2) * 4);
   }
   if (lat_scratch_bytes_ && !(lat_scratch_ = (float*)dalloc(lat_scratch_bytes_))) return false;
-  if (want_h32 && (!(h32_ = (float*)dalloc(T * W * 4)) || !(id_weight_ = (float*)dalloc(T * 4)))) return false;
+  if (nmix && !(mix_ = dalloc(nmix * T * W * es_))) return false;
+  if (want_h32 && ((block_ != 3 && !(h32_ = (float*)dalloc(T * W * 4))) || !(id_weight_ = (float*)dalloc(T * 4)))) return false;
   const size_t P = T * std::max<size_t>(top, 1);
   if (!(pair_expert_ = (int*)dalloc(P * 4)) || !(pair_weight_ = (float*)dalloc(P * 4)) || !(gate_ = (float*)dalloc(T * 4)) ||
       !(row_token_ = (int*)dalloc((size_t)max_rows_ * 4)) || !(row_pair_ = (int*)dalloc((size_t)max_rows_ * 4)) ||
@@ -990,11 +1074,11 @@ bool StackModel::expert_pair(const void* a, int lda, const void* w_gu, int64_t g
                              float* out, int64_t stream, int act) {
   const int W = width_;
   StkGemmArgs g;
-  g.a = a, g.lda = lda, g.w = w_gu, g.w_group_stride = gu_stride, g.M = rows, g.N = (act == 3 ? 1 : 2) * fp, g.K = W;
+  g.a = a, g.lda = lda, g.w = w_gu, g.w_group_stride = gu_stride, g.M = rows, g.N = (act >= 3 ? 1 : 2) * fp, g.K = W;
   g.tile_group = tile_group, g.granule = granule, g.a_row = a_row, g.a_scale = a_scale;
   g.limit = limit, g.act = act;
   const bool fused = dt_ == VRA_BF16 && W % 8 == 0 && lda % 8 == 0;
-  if (act == 3) {  // no gate: an element-wise activation, in the epilogue whatever the type
+  if (act >= 3) {  // no gate: an element-wise activation, in the epilogue whatever the type
     g.epi = 2, g.out = act_, g.ldo = fp;
     vra_stack_gemm(g, dt_, stream);
   } else if (fused) {
@@ -1163,7 +1247,7 @@ bool StackModel::forward(const InputMetadata& md, int64_t stream, uint32_t* toke
     }
     trace_bytes_ = need_b;
   }
-  if (block_ == 2) {
+  if (block_ >= 2) {
     if (!forward_sandwich(md, stream)) return false;
   } else {
     vra_stack_embed_sinpos(md.input_ids, md.positions, embed_, pos_kind_ == 0 ? inv_freq_ : nullptr, x_, T, W, vocab_, dt_, stream);
@@ -1171,7 +1255,7 @@ bool StackModel::forward(const InputMetadata& md, int64_t stream, uint32_t* toke
   }
   // sequential blocks: the output of a sub-block is added to the residual inside the launch of the next norm (`pending`)
   const float* pending = nullptr;
-  for (size_t li = 0; li < layers_.size() && block_ != 2; li++) {
+  for (size_t li = 0; li < layers_.size() && block_ < 2; li++) {
     const StackLayer& L = layers_[li];
     if (block_ == 0) {
       // h = norm(x); a mixture-of-experts layer's router (and its shared expert's gate) reads h inside the same launch
@@ -1238,9 +1322,9 @@ bool StackModel::forward(const InputMetadata& md, int64_t stream, uint32_t* toke
 // ---------------------------------------------------------------------------------------------
 // the recurrence has left o (f32 [T, heads * vdim]) in ro_: per-head norm, gate, output projection -> out (f32 [T, width])
 bool StackModel::recurrent_tail(const StackLayer& L, const InputMetadata& md, const float* gate, int gate_ld, int gate_act, const void* w_o, float* out,
-                                int64_t stream) {
+                                int64_t stream, int w_per_head) {
   const int T = md.n_tokens, H = L.s_heads(), V = L.s_vdim();
-  vra_stack_head_norm_gate(ro_, L.out_norm_w, gate, gate_ld, gate_act, eps_, attn_, T, H, V, dt_, stream);
+  vra_stack_head_norm_gate(ro_, L.out_norm_w, gate, gate_ld, gate_act, eps_, attn_, T, H, V, dt_, stream, w_per_head);
   StkGemmArgs o;
   o.a = attn_, o.lda = H * V, o.w = w_o, o.M = T, o.N = width_, o.K = H * V, o.out = out, o.ldo = width_, o.out_f32 = 1;
   vra_stack_gemm(o, dt_, stream);
@@ -1378,30 +1462,35 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
   vra_stack_embed_pair(e, dt_, stream);
   if (take_stack_err(error, "embedding")) return false;
   StkSandwichArgs pend;  // the parts of the last sub-block's output, not yet normed and added (post_w null: none)
-  auto seam = [&](const float* pre_w, const float* pre_b, float pre_alpha, const StackLayer* router) {
+  // post blocks: the next sub-block reads the residual stream itself (`reads`: it takes the row in the model's type)
+  auto seam = [&](const float* pre_w, const float* pre_b, float pre_alpha, const StackLayer* router, bool reads = false) {
     StkSandwichArgs s = pend;
+    s.pre_identity = block_ == 3 && reads;
     s.x = x_, s.pre_w = pre_w, s.pre_b = pre_b, s.pre_alpha = pre_alpha, s.norm_kind = norm_kind_, s.h = h_, s.eps = eps_, s.T = T, s.W = W;
     if (router) {
       s.router_w = router->router, s.router_bias = router->router_bias, s.n_router = router->experts + router->n_identity, s.top = router->top;
       s.pair_expert = pair_expert_, s.pair_weight = pair_weight_;
       if (router->router_kind >= 2) {
         s.router_kind = router->router_kind - 1, s.n_groups = router->n_groups, s.keep = router->keep, s.n_identity = router->n_identity;
-        if (router->n_identity > 0) s.h32 = h32_, s.id_weight = id_weight_;
+        s.weight_scale = router->router_scale;
+        if (router->n_identity > 0) s.h32 = block_ == 3 ? nullptr : h32_, s.id_weight = id_weight_;
       }
     }
-    if (s.post_w || s.pre_w) vra_stack_sandwich_norm(s, dt_, stream);
+    if (s.post_w || s.pre_w || s.pre_identity) vra_stack_sandwich_norm(s, dt_, stream);
     pend = StkSandwichArgs();
     return !take_stack_err(error, "norm");
   };
   for (size_t li = 0; li < layers_.size(); li++) {
     const StackLayer& L = layers_[li];
-    if (!seam(L.norm_w, L.norm_b, L.norm_alpha, nullptr)) return false;
+    if (!seam(L.norm_w, L.norm_b, L.norm_alpha, nullptr, L.mixer != 8)) return false;  // (wkv takes its mixes from the f32 rows)
     bool ok = false;
     switch (L.mixer) {
       case 1: ok = mixer_latent(L, md, stream); break;
       case 3: ok = mixer_delta(L, md, stream); break;
       case 4: ok = mixer_retention(L, md, stream); break;
       case 6: ok = mixer_lightning(L, md, stream); break;
+      case 7: ok = mixer_differential(L, md, stream); break;
+      case 8: ok = mixer_wkv(L, md, stream); break;
       default: ok = L.right_kind == 1 ? mixer_hybrid(L, md, stream) : mixer_parallel(L, md, stream); break;
     }
     if (!ok) return false;
@@ -1411,7 +1500,7 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
       if (L.branch_norm) pend.p1_norm_w = L.left_out_w, pend.p2_norm_w = L.right_out_w;
     }
     if (L.mlp == 2) {
-      if (!seam(L.norm2_w, L.norm2_b, L.norm2_alpha, &L)) return false;
+      if (!seam(L.norm2_w, L.norm2_b, L.norm2_alpha, &L, true)) return false;
       const int P = T * L.top;
       const int granule = vra_stack_gemm_granule(P, L.experts);
       const int rows = round_up(P + L.experts * (granule - 1), granule);
@@ -1424,12 +1513,22 @@ bool StackModel::forward_sandwich(const InputMetadata& md, int64_t stream) {
         return false;
       pend.p1 = pair_out_, pend.n1 = L.top, pend.pw = L.router_kind >= 1 ? pair_weight_ : nullptr;
       pend.post_w = L.post2_w, pend.post_b = L.post2_b, pend.post_alpha = L.post2_alpha;
-      if (L.router_kind == 2 && L.n_identity > 0) {  // an identity expert's pair has no row: its weight times the feed-forward's own input
+      if (block_ == 3) {  // identity experts hand back the residual row itself: their summed weight times the row the sum is added to
+        if (L.n_identity > 0) pend.pe = pair_expert_, pend.xw = id_weight_;
+        if (L.shared_ff > 0) {
+          if (!expert_pair(h_, W, L.s_gu, 0, L.s_down, 0, T, L.sffp, L.shared_ff, L.shared_limit, nullptr, 0, nullptr, nullptr, nullptr, sh_, stream, L.act_kind)) return false;
+          pend.p2 = sh_, pend.c2 = 1.f;
+        }
+      } else if (L.router_kind == 2 && L.n_identity > 0) {  // an identity expert's pair has no row: its weight times the feed-forward's own input
         pend.pe = pair_expert_, pend.p2 = h32_, pend.p2w = id_weight_, pend.c2 = 1.f;
       } else if (L.shared_ff > 0) {  // the shared expert runs for every token and is added as it is
         if (!expert_pair(h_, W, L.s_gu, 0, L.s_down, 0, T, L.sffp, L.shared_ff, L.shared_limit, nullptr, 0, nullptr, nullptr, nullptr, sh_, stream, L.act_kind)) return false;
         pend.p2 = sh_, pend.c2 = 1.f;
       }
+    } else if (L.mlp == 5) {
+      if (!seam(nullptr, nullptr, 1.f, nullptr, true)) return false;
+      if (!expert_pair(h_, W, L.s_gu, 0, L.s_down, 0, T, L.sffp, L.ff, 0.f, nullptr, 0, nullptr, nullptr, nullptr, pair_out_, stream, 4)) return false;
+      pend.p1 = pair_out_, pend.n1 = 1, pend.post_w = L.post2_w;
     } else if (L.mlp == 4) {
       if (!seam(L.norm2_w, L.norm2_b, L.norm2_alpha, nullptr)) return false;
       if (!expert_pair(h_, W, L.s_gu, 0, L.s_down, 0, T, L.sffp, L.ff, L.limit, nullptr, 0, nullptr, nullptr, nullptr, pair_out_, stream, 0)) return false;
@@ -1461,6 +1560,60 @@ bool StackModel::mixer_lightning(const StackLayer& L, const InputMetadata& md, i
   o.a = attn_, o.lda = H * V, o.w = L.o, o.M = T, o.N = W, o.K = H * V, o.out = o_, o.ldo = W, o.out_f32 = 1;
   vra_stack_gemm(o, dt_, stream);
   return !take_stack_err(error, "lightning");
+}
+
+// differential attention: q (| k | v) in one launch (biases in its epilogue, f32), per-head norms of q and k in the launch that writes the
+// cache rows, both maps and their combination in the attention launch, output projection with its bias
+bool StackModel::mixer_differential(const StackLayer& L, const InputMetadata& md, int64_t stream) {
+  const int T = md.n_tokens, W = width_, n1 = L.nqkv(), H = L.heads, lq = L.nq(), lk = L.nk(), lv = L.nv();
+  StkGemmArgs p;
+  p.a = h_, p.lda = W, p.w = L.qkv, p.bias = L.qkv_bias, p.M = T, p.N = n1, p.K = W, p.out = z_, p.ldo = n1, p.out_f32 = 1;
+  vra_stack_gemm(p, dt_, stream);
+  StkHeadPrepArgs hp;
+  hp.raw = z_, hp.ld = n1, hp.Hq = 2 * H, hp.dim = L.dim, hp.qn_w = L.qn_w, hp.eps = eps_, hp.positions = md.positions, hp.q_out = qkv_, hp.q_ld = lq, hp.T = T;
+  if (L.owns_cache) {
+    hp.k_off = lq, hp.v_off = lq + lk, hp.Hk = 2 * L.kv_heads, hp.nv = lv, hp.kn_w = L.kn_w, hp.slots = md.slot_mapping;
+    hp.k_out = kc_[L.cache], hp.k_ld = lk, hp.v_out = vc_[L.cache], hp.v_ld = lv;
+  }
+  vra_stack_head_prep(hp, dt_, stream);
+  StkAttnArgs a;
+  a.q = qkv_, a.ldq = lq, a.out = attn_, a.kc = kc_[L.cache], a.vc = vc_[L.cache];
+  a.positions = md.positions, a.block_tables = md.block_tables, a.context_lens = md.context_lens;
+  a.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr;
+  a.B = md.n_seqs, a.T = T, a.max_q = md.is_prefill ? md.max_seqlen_q : 1, a.H = H, a.G = L.kv_heads, a.dim = L.dim, a.vdim = L.vdim;
+  a.BS = ec_.block_size, a.max_blocks = md.max_blocks, a.scale = L.scale;
+  a.maps = 2, a.diff_lambda = L.lambda, a.diff_eps = eps_, a.diff_scale = 1.f - L.diff;
+  vra_stack_attention(a, dt_, stream);
+  StkGemmArgs o;
+  o.a = attn_, o.lda = H * L.vdim, o.w = L.o, o.bias = L.o_bias, o.M = T, o.N = W, o.K = H * L.vdim, o.out = o_, o.ldo = W, o.out_f32 = 1;
+  vra_stack_gemm(o, dt_, stream);
+  return !take_stack_err(error, "differential attention");
+}
+
+// time mixing: the five shifted mixes in one launch (which also moves the carried row on), r | k | v | gate as four products of one launch
+// (f32), the decay's two low-rank stages with tanh and exp(-exp) in their epilogues, the recurrence with the bonus, norm + gate, o
+bool StackModel::mixer_wkv(const StackLayer& L, const InputMetadata& md, int64_t stream) {
+  const int T = md.n_tokens, W = width_, H = L.heads, D = L.dim, n = H * D, n1 = 4 * n, R = L.rank_a;
+  StkShiftArgs sh;
+  sh.x = x_, sh.mu = L.mu, sh.n = 5, sh.shift_state = L.conv_state, sh.positions = md.positions, sh.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr;
+  sh.state_slots = md.state_slots, sh.out = mix_, sh.T = T, sh.B = md.n_seqs, sh.W = W;
+  vra_stack_token_shift(sh, dt_, stream);
+  StkGemmArgs p;
+  p.a = mix_, p.lda = W, p.a_batch_stride = (int64_t)T * W, p.w = L.qkv, p.w_batch_stride = (int64_t)n * W, p.batch = 4, p.M = T, p.N = n, p.K = W;
+  p.out = z_, p.ldo = n1, p.out_batch_stride = n, p.out_f32 = 1;
+  vra_stack_gemm(p, dt_, stream);
+  StkGemmArgs l1;
+  l1.a = (const char*)mix_ + (size_t)4 * T * W * es_, l1.lda = W, l1.w = L.lr1, l1.M = T, l1.N = R, l1.K = W, l1.out = act_, l1.ldo = R, l1.epi = 2, l1.act = 5;
+  vra_stack_gemm(l1, dt_, stream);
+  StkGemmArgs l2;
+  l2.a = act_, l2.lda = R, l2.w = L.lr2, l2.bias = L.lr2_bias, l2.M = T, l2.N = n, l2.K = R, l2.out = z2_, l2.ldo = n, l2.out_f32 = 1, l2.epi = 2, l2.act = 6;
+  vra_stack_gemm(l2, dt_, stream);
+  StkScanArgs sc;
+  sc.q = z_, sc.ldq = n1, sc.k = z_ + n, sc.ldk = n1, sc.v = z_ + 2 * n, sc.ldv = n1, sc.decay = z2_, sc.ldd = n, sc.bonus = L.bonus;
+  scan_common(sc, L, md, ro_);
+  vra_stack_linear_scan(sc, stream);
+  if (take_stack_err(error, "wkv")) return false;
+  return recurrent_tail(L, md, z_ + 3 * n, n1, 1, L.o, o_, stream, 1);
 }
 
 // two branches on one input, each with a norm of its own in the seam that follows.  Left: softmax attention over the paged cache (biases

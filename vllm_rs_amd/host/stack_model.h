@@ -6,6 +6,8 @@
 //           sandwich:    x <- x + norm1b(mixer(norm1(x))),  x <- x + norm2b(ff(norm2(x)))   (Zifetar: RMS norms, norm_offset added to the weights;
 //                        Sudosun: Dynamic Tanh norms, the head is the embedding table;
 //                        Pesivik: layer norms, layer_scale: each sub-block's normed output times one factor per channel)
+//           post:        x <- x + norm1(mixer(x)),  x <- x + norm2(ff(x)): a sub-block reads the residual stream itself and only its output has a
+//                        norm (Kemavik: RMS norms, norm_offset added to the weights)
 //   norm    rms: RMS norm over `groups` equal parts of the width;  dyt: Dynamic Tanh  tanh(alpha x) w + b  (no statistics);
 //           layer: (x - mean) / sqrt(variance + eps) w  (sandwich blocks)
 //   pos     sinusoid: a position vector added to the embedding;  none: positions enter inside the mixers
@@ -32,13 +34,22 @@
 //                      head, a sigmoid output gate per head and rotary on neighbouring pairs (YaRN-scaled); the right branch is a gelu branch
 //                      times a real-gated diagonal recurrence behind a short convolution (block-diagonal gates); each branch's output has an
 //                      RMS norm of its own over the width (branch_norm=1) before the scaled sum
+//           differential: causal softmax attention whose query and key heads hold two maps; both maps weigh the same values and the second's
+//                      output is taken off lambda times (lambda: one number a layer from four vectors and `diff`), then an RMS norm per head
+//                      without weight times 1 - diff; biases, per-head q / k norm, no rotation, grouped key/value heads, optionally another
+//                      layer's keys / values (kv_from)
+//           wkv:       time mixing: the inputs of r, k, v, gate and decay are mixes of a token's row with the row before it (token shift), a
+//                      matrix state per head with a decay per key channel exp(-exp(w0 + W_w2 tanh(W_w1 .))), a bonus for the current token,
+//                      per-head output norm with a weight over all heads' channels, silu gate
 //   mlp     none | dense (PolyNorm activation) | moe (sigmoid router, clamped gated experts, gated shared expert) | gated (gelu_tanh(gate) * up)
 //           | clamped (dense, the clamped gated form of the experts above);  moe with router=softmax_all: scores are a softmax over all
 //           router outputs, a correction is added for the choice only, the choice is restricted to the best `keep` of `groups` groups of
 //           neighbouring experts, the weights are the plain scores, and the last `identity` outputs are experts that return their input;
 //           moe with router=sigmoid_norm: sigmoid scores, the correction and the groups as before (a group's worth is the sum of its two best
 //           corrected scores), weights = the chosen scores divided by their sum; a shared expert may run beside it, added as it is;
+//           relu2 (dense, squared relu, no gate);
 //           act=gelu: experts (and the shared one) without a gate, down(gelu(up h)) with the exact (erf) gelu
+//           post blocks: router=softmax_all with router_scale (a constant on all weights) and a shared expert added as it is
 //   logit_softcap: logits <- cap * tanh(logits / cap)
 //   sandwich blocks with norm=dyt use Dynamic Tanh for all four norms of a layer; tie_head=1: the head is the embedding table
 //   weights_of=j: the layer runs with layer j's tensors and a cache of its own
@@ -55,9 +66,10 @@
 //         conv=.. rank_a=.. rank_g=.. decay=d0,d1,.. chunk=.. qk_norm=0|1 bias=0|1 rs_factor=.. rs_low=.. rs_high=.. rs_original=..
 //         r_heads=.. r_dim=.. r_vdim=.. tau=.. left_scale=.. right_scale=..
 //         lowrank=0|1 right=gla|rglru r_width=.. r_blocks=.. r_conv=.. head_temp=0|1 head_gate=0|1 branch_norm=0|1
+//         diff=.. (differential)
 //         rot_layout=half|pairs (latent: pairs unless given, the other mixers: half)
-//         mlp=none|dense|moe|gated|clamped ff=.. experts=.. top=.. limit=.. shared_ff=.. shared_limit=.. router=sigmoid|softmax|softmax_all|sigmoid_norm
-//         act=clamped|silu|gelu identity=.. groups=.. keep=..
+//         mlp=none|dense|moe|gated|clamped|relu2 ff=.. experts=.. top=.. limit=.. shared_ff=.. shared_limit=.. router=sigmoid|softmax|softmax_all|sigmoid_norm
+//         act=clamped|silu|gelu identity=.. groups=.. keep=.. router_scale=..
 #pragma once
 #include <map>
 #include <string>
@@ -69,7 +81,7 @@ namespace vra {
 
 struct StackLayer {
   // mixer: 0 softmax attention, 1 latent attention, 2 sigmoid attention, 3 gated delta rule, 4 retention, 5 parallel (softmax attention
-  // beside a gated linear attention or a real-gated diagonal recurrence), 6 lightning
+  // beside a gated linear attention or a real-gated diagonal recurrence), 6 lightning, 7 differential attention, 8 wkv
   int mixer = 0;
   int heads = 0, kv_heads = 0, dim = 0, vdim = 0, temp_every = 0, kv_from = -1, weights_of = -1;
   float scale = 1.f, softcap = 0.f, temp_coef = 0.f;
@@ -91,9 +103,14 @@ struct StackLayer {
   // of r_width channels with r_blocks gate blocks behind a convolution of `conv` taps; the left branch's per-head temperature and output
   // gate, rotary layout (1 = neighbouring pairs), a norm per branch before the sum
   int lowrank = 1, right_kind = 0, r_width = 0, r_blocks = 1, head_temp = 0, head_gate = 0, rot_layout = 0, branch_norm = 0;
+  // differential attention: maps per head, the constant part of lambda, lambda itself (from the tensors);  wkv: width of the shifted row
+  int maps = 1, shift_w = 0;
+  float diff = 0.f, lambda = 0.f;
+  float router_scale = 1.f;  // router_kind 2: multiplies the weights
   // router_kind 2 / 3: identity experts (2) and expert groups
   int n_identity = 0, n_groups = 0, keep = 0;
-  // feed-forward: 0 none, 1 dense (PolyNorm), 2 mixture of experts, 3 gated dense (gelu_tanh(gate) * up), 4 clamped gated dense
+  // feed-forward: 0 none, 1 dense (PolyNorm), 2 mixture of experts, 3 gated dense (gelu_tanh(gate) * up), 4 clamped gated dense, 5 dense with a
+  // squared relu
   int mlp = 0, ff = 0, experts = 0, top = 0, shared_ff = 0;
   float limit = 0.f, shared_limit = 0.f;
   // mixture of experts: router 0 = sigmoid scores as weights on the experts' inputs, 1 = biased logits, softmax over the chosen ones, weights
@@ -105,26 +122,26 @@ struct StackLayer {
   int cache = -1;          // index of the paged cache this layer reads (its own, or the one of layer kv_from)
   bool owns_cache = false;
   int ffp = 0, sffp = 0;   // expert / shared (or gated dense) widths rounded up to 16 (zero rows and columns)
-  int nq() const { return heads * (mixer == 1 ? dim + rot_dim : dim); }
-  int nk() const { return kv_heads * dim; }
+  int nq() const { return heads * (mixer == 1 ? dim + rot_dim : maps * dim); }
+  int nk() const { return kv_heads * maps * dim; }
   int nv() const { return kv_heads * vdim; }
   // columns of the joint input projection: q (| k | v) of softmax attention, q | k | v | gate of sigmoid attention, the three latents (| head gates)
   int nqkv() const {
     if (mixer == 1) return q_rank + kv_rank + rot_dim + (head_gate ? heads : 0);
     if (mixer == 2) return nq() + nk() + nv() + heads * vdim;
     if (mixer == 3) return 2 * nk() + heads * vdim + heads + (lowrank ? 0 : heads + heads * vdim);  // q | k (kv_heads each) | v | write strengths (| decays | gate)
-    if (mixer == 4 || mixer == 6) return 2 * heads * dim + 2 * heads * vdim;       // q | k | v | gate
+    if (mixer == 4 || mixer == 6 || mixer == 8) return 2 * heads * dim + 2 * heads * vdim;  // q | k | v | gate
     if (mixer == 5 && right_kind == 1) return nq() + nk() + nv() + (head_gate ? heads : 0) + 2 * r_width;  // left q | k | v | gates, right gelu branch | recurrent branch
     if (mixer == 5) return nq() + nk() + nv() + r_heads * (2 * r_dim + 2 * r_vdim);  // left q | k | v, right q | k | v | gate
     return nq() + (owns_cache ? nk() + nv() : 0);
   }
-  bool has_cache() const { return mixer != 3 && mixer != 4 && mixer != 6; }
+  bool has_cache() const { return mixer != 3 && mixer != 4 && mixer != 6 && mixer != 8; }
   // the recurrent part: heads, key and value sizes of the matrix state (0 heads: none)
-  int s_heads() const { return mixer == 5 ? (right_kind == 1 ? 0 : r_heads) : (mixer == 3 || mixer == 4 || mixer == 6 ? heads : 0); }
+  int s_heads() const { return mixer == 5 ? (right_kind == 1 ? 0 : r_heads) : (mixer == 3 || mixer == 4 || mixer == 6 || mixer == 8 ? heads : 0); }
   int vec_state() const { return mixer == 5 && right_kind == 1 ? r_width : 0; }  // a diagonal recurrence: one state value per channel
   int s_dim() const { return mixer == 5 ? r_dim : dim; }
   int s_vdim() const { return mixer == 5 ? r_vdim : vdim; }
-  int conv_channels() const { return mixer == 3 ? 2 * nk() + heads * vdim : vec_state(); }
+  int conv_channels() const { return mixer == 3 ? 2 * nk() + heads * vdim : (mixer == 8 ? shift_w : vec_state()); }  // (wkv keeps one row: conv = 2)
   // elements of one token's cache rows
   int k_row() const { return mixer == 1 ? kv_rank + rot_dim : nk(); }
   int v_row() const { return mixer == 1 ? 0 : nv(); }
@@ -133,6 +150,7 @@ struct StackLayer {
   float *norm_b = nullptr, *norm2_w = nullptr, *norm2_b = nullptr;  // Dynamic Tanh: offsets, and the second norm of a sequential block
   float norm_alpha = 1.f, norm2_alpha = 1.f;
   void* qkv = nullptr;     // [nqkv(), width]
+  float *mu = nullptr, *bonus = nullptr, *o_bias = nullptr;  // wkv: shift mixes f32 [5, width] (r, k, v, gate, decay), bonus f32 [heads, dim];  differential: f32 [width]
   float* qkv_bias = nullptr;  // sigmoid attention: f32 [nqkv()] (zeros for the gate rows)
   void* o = nullptr;       // [width, heads * vdim]
   void* uq = nullptr;      // latent: [heads * (dim + rot_dim), q_rank]
@@ -216,7 +234,10 @@ class StackModel : public ModelBase {
   bool mixer_parallel(const StackLayer& L, const InputMetadata& md, int64_t stream);
   bool mixer_lightning(const StackLayer& L, const InputMetadata& md, int64_t stream);
   bool mixer_hybrid(const StackLayer& L, const InputMetadata& md, int64_t stream);
-  bool recurrent_tail(const StackLayer& L, const InputMetadata& md, const float* gate, int gate_ld, int gate_act, const void* w_o, float* out, int64_t stream);
+  bool mixer_differential(const StackLayer& L, const InputMetadata& md, int64_t stream);
+  bool mixer_wkv(const StackLayer& L, const InputMetadata& md, int64_t stream);
+  bool recurrent_tail(const StackLayer& L, const InputMetadata& md, const float* gate, int gate_ld, int gate_act, const void* w_o, float* out, int64_t stream,
+                      int w_per_head = 0);
   bool forward_sandwich(const InputMetadata& md, int64_t stream);
   void rotary_table(StackLayer& L);
   float* upload_floats(const std::vector<float>& v);
@@ -230,7 +251,7 @@ class StackModel : public ModelBase {
   int dt_ = 0;
   size_t es_ = 2;
   int width_ = 0, vocab_ = 0, groups_ = 1;
-  int block_ = 0, norm_kind_ = 0, pos_kind_ = 0;  // 0 parallel / rms / sinusoid, 1 sequential / dyt / none, block 2 sandwich, norm 2 layer norm
+  int block_ = 0, norm_kind_ = 0, pos_kind_ = 0;  // 0 parallel / rms / sinusoid, 1 sequential / dyt / none, block 2 sandwich, 3 post, norm 2 layer norm
   float norm_offset_ = 0.f, embed_scale_ = 1.f;    // added to every norm weight at load; multiplies the embedding row
   int embed_norm_ = 0, pair_buckets_ = 0, tie_head_ = 0, layer_scale_ = 0;
   float logit_softcap_ = 0.f;
@@ -260,6 +281,7 @@ class StackModel : public ModelBase {
   // activations
   int max_tokens_ = 0, max_seqs_ = 0, logit_rows_cap_ = 0, max_rows_ = 0;
   float *x_ = nullptr, *o_ = nullptr, *z_ = nullptr, *pair_out_ = nullptr, *sh_ = nullptr, *xl_ = nullptr, *logits_ = nullptr;
+  void* mix_ = nullptr;  // wkv: the shifted mixes [5, T, width]
   void *h_ = nullptr, *qkv_ = nullptr, *attn_ = nullptr, *act_ = nullptr, *hl_ = nullptr, *qa_ = nullptr;
   int *pair_expert_ = nullptr, *row_token_ = nullptr, *row_pair_ = nullptr, *tile_group_ = nullptr;
   float *pair_weight_ = nullptr, *row_scale_ = nullptr, *gate_ = nullptr;
