@@ -737,7 +737,7 @@ void vra_stack_op_linear_scan_ex(const float* q, int32_t ldq, const float* k, in
 /* attention_latent: the softmax attention over a latent cache (csrc/stack_latent.hip): one row of k_ld elements per token, keys = its first
  * `dim` columns for every head, values = its first vdim columns; window, sink, head_scale, gate as in attention_window.  Decode form
  * (cu_q null) with scratch: B * splits * H * (vdim + 2) floats, the key range in `splits` parts.
- * gemm_post: vra_stack_op_gemm with bias and the element-wise epilogues: epi 2 = act(alpha sum + bias) (act 3: exact gelu),
+ * gemm_post: vra_stack_op_gemm with bias and the element-wise epilogues: epi 2 = act(alpha sum + bias) (act 3: exact gelu, 4: max(z, 0)^2, 5: tanh, 6: exp(-exp z)),
  * softcap > 0: softcap tanh(v / softcap). */
 void vra_stack_op_attention_latent(const void* q, int32_t ldq, void* out, const void* cache, int32_t k_ld, const int64_t* positions,
                                    const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_q, int32_t B, int32_t T,
@@ -748,6 +748,33 @@ void vra_stack_op_gemm_post(const void* a, int32_t lda, const void* w, int64_t w
                             int32_t M, int32_t N, int32_t K, float alpha, const float* bias, const int32_t* tile_group, int32_t granule,
                             const int32_t* a_row, const int32_t* out_row, int32_t epi, int32_t act, float softcap, int32_t dtype,
                             int64_t stream);
+
+/* attention_differential: causal softmax attention with two maps per head over the paged cache: q rows [map 1 | map 2] per head (dim each), K rows
+ * the same per key/value head, V rows vdim per key/value head; with a1, a2 the maps' outputs o = a1 - lambda a2,
+ * out = o / sqrt(mean(o^2) + eps) * out_scale.  Decode form (cu_q null) with scratch: B * splits * H * 2 * (vdim + 2) floats, the key range in
+ * `splits` parts (scratch null: one launch).
+ * token_shift: out[m, t] = x[t] + (x[t - 1] - x[t]) mu[m] for n mixes; the row before a step's first from shift_state [slots, W], which moves on.
+ * bonus_scan: the linear recurrence with per-channel decays whose output reads the state before the decay,
+ * o = (S + diag(bonus) k v^T)^T (q_scale q); S <- diag(decay) S + k v^T  (state [slots, H, vdim, dim] f32).
+ * head_norm_gate: out = o / sqrt(mean(o^2) + eps) * w * act(gate) per head (w [vdim], or [H, vdim] with w_per_head; gate_act 1 silu, 2 sigmoid).
+ * seam_post: x += N(sum_j pw p1 + p2 + xw x; post_w) (RMS norm), h = x in dtype, and the router of kind 1 on x with weight_scale on all weights. */
+void vra_stack_op_attention_differential(const void* q, int32_t ldq, void* out, const void* kc, const void* vc, const int64_t* positions,
+                                         const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_q, int32_t B,
+                                         int32_t T, int32_t max_q, int32_t H, int32_t G, int32_t dim, int32_t vdim, int32_t BS,
+                                         int32_t max_blocks, float scale, float lambda, float eps, float out_scale, float* scratch,
+                                         int64_t scratch_bytes, int32_t splits, int32_t dtype, int64_t stream);
+void vra_stack_op_token_shift(const float* x, const float* mu, int32_t n, float* shift_state, const int64_t* positions, const uint32_t* cu_q,
+                              const int32_t* state_slots, void* out, int32_t T, int32_t B, int32_t W, int32_t dtype, int64_t stream);
+void vra_stack_op_bonus_scan(const float* q, int32_t ldq, const float* k, int32_t ldk, const float* v, int32_t ldv, const float* decay,
+                             int32_t ldd, const float* bonus, float q_scale, float* state, const int32_t* state_slots,
+                             const int64_t* positions, const uint32_t* cu_q, float* out, int32_t ldo, int32_t B, int32_t H, int32_t qk_rep,
+                             int32_t dim, int32_t vdim, int64_t stream);
+void vra_stack_op_head_norm_gate(const float* o, const float* w, int32_t w_per_head, const float* gate, int32_t gate_ld, int32_t gate_act, float eps,
+                                 void* out, int32_t T, int32_t H, int32_t vdim, int32_t dtype, int64_t stream);
+void vra_stack_op_seam_post(float* x, const float* p1, int32_t n1, const float* pw, const int32_t* pe, const float* p2, const float* xw,
+                            const float* post_w, void* h, float eps, int32_t T, int32_t W, const void* router_w, const float* router_bias,
+                            int32_t n_router, int32_t top, int32_t n_identity, float weight_scale, int32_t* pair_expert, float* pair_weight,
+                            float* id_weight, int32_t dtype, int64_t stream);
 
 /* decode-step microbenchmark hook used by bench.py: runs `steps` decode steps of the current
  * running batch back to back (graph replay when enabled) and returns elapsed ms measured with HIP

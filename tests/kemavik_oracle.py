@@ -119,7 +119,7 @@ def route(h, router, w, p):
     z = h @ w[p + "router"].T
     e = np.exp(z - z.max(-1, keepdims=True))
     s = e / e.sum(-1, keepdims=True)
-    chosen = np.argsort(-(s + w[p + "correction"]), axis=-1, kind="stable")[:, :int(router["top"])]
+    chosen = np.argsort(-(s + w[p + "correction"]), axis=-1, kind="stable")[:, :int(router.get("top", 1))]
     return chosen, np.take_along_axis(s, chosen, -1) * float(router.get("scale", 1.0))
 
 

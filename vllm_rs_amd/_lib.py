@@ -233,6 +233,12 @@ def load():
          P, P, P, c_i32, P, c_i64, c_i32, c_i32, c_i64)
     _sig(lib, "vra_stack_op_gemm_post", None, P, c_i32, P, c_i64, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_f32, P, P, c_i32, P, P, c_i32, c_i32, c_f32,
          c_i32, c_i64)
+    _sig(lib, "vra_stack_op_attention_differential", None, P, c_i32, P, P, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32,
+         c_f32, c_f32, c_f32, c_f32, P, c_i64, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_token_shift", None, P, P, c_i32, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_bonus_scan", None, P, c_i32, P, c_i32, P, c_i32, P, c_i32, P, c_f32, P, P, P, P, P, c_i32, c_i32, c_i32, c_i32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_head_norm_gate", None, P, P, c_i32, P, c_i32, c_i32, c_f32, P, c_i32, c_i32, c_i32, c_i32, c_i64)
+    _sig(lib, "vra_stack_op_seam_post", None, P, P, c_i32, P, P, P, P, P, P, c_f32, c_i32, c_i32, P, P, c_i32, c_i32, c_i32, c_f32, P, P, P, c_i32, c_i64)
     _sig(lib, "vra_engine_create_spec", P, MC, EC, C.c_char_p)
     _sig(lib, "vra_engine_replay_step", c_i32, P, c_i32, P, P, P, P, P, c_i32, P, P)
     _sig(lib, "vra_engine_debug_layer_trace", None, P, c_i32)

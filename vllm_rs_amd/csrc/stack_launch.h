@@ -120,12 +120,14 @@ struct StkAttnArgs {
   // everything up to the store in f32.  Causal mask, scale and sizes as above; no sink, gate, chunk, window, cap or temperature beside it.
   int maps = 1;
   float diff_lambda = 0.f, diff_eps = 0.f, diff_scale = 1.f;
-  // latent decode form: f32 scratch of B * splits * H * (vdim + 2) floats for the parts of the key range (null: the one-launch kernel)
+  // latent and differential decode forms: f32 scratch of B * splits * H * maps * (vdim + 2) floats for the parts of the key range (null: the one-launch kernel)
   float* scratch = nullptr;
   size_t scratch_bytes = 0;
   int splits = 0;
 };
 void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream);
+// parts of the key range the differential decode form takes (a model's constants: it fixes the order of the sums)
+int vra_stack_diff_splits(int max_len, int max_seqs, int heads, int vdim);
 // its shared-row form on the matrix cores (stack_latent.hip): bf16 prompt steps with G = 1 and vc = kc, rows up to 576 wide, values up to 512;
 // false: not a shape of that kernel, nothing was launched
 // vra_stack_latent_decode: the same for one token per sequence, in two launches over `splits` parts of the key range (any number from 1 to 64; it

@@ -898,7 +898,8 @@ __global__ __launch_bounds__(256 * MAPS) void stk_attn_prefill_mfma_kernel(StkAt
 // One decoded token per sequence: a workgroup per (sequence, query head); its 8 waves take the 64-key tiles of the context in turn,
 // read K rows straight from the cache (lane = key, 16 bytes a load where the row allows) and V rows channel-wise (lane = channel), and
 // meet once in LDS.  The order of the sums depends on the context length alone.
-// MAPS 2: the differential form of StkAttnArgs (both maps' scores of a key, then one pass over the values for both).
+// MAPS 2: the differential form of StkAttnArgs (both maps' scores of a key, then one pass over the values for both);
+// with scratch the key tiles are spread over gridDim.z workgroups and stk_attn_decode_join_kernel adds their parts.
 #define STK_DW 8
 template <typename T>
 __device__ __forceinline__ float stk_dot_row(const float* qs, const T* kr, int dim) {
@@ -961,7 +962,7 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
   int key_lo = a.chunk > 0 ? (int)(p / a.chunk * a.chunk) : 0;
   if (a.window > 0) key_lo = max(key_lo, (int)(p - a.window + 1));
   const float hscale = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
-  for (int kt0 = key_lo / 64 * 64 + wave * 64; kt0 < n_keys; kt0 += STK_DW * 64) {
+  for (int kt0 = key_lo / 64 * 64 + (wave * (int)gridDim.z + (int)blockIdx.z) * 64; kt0 < n_keys; kt0 += STK_DW * (int)gridDim.z * 64) {
     const int key = kt0 + lane;
     float s[MAPS], corr[MAPS];
     for (int mp = 0; mp < MAPS; mp++) s[mp] = -INFINITY;
@@ -1050,6 +1051,28 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
   __syncthreads();
   T* out = (T*)a.out + (size_t)b * a.H * vdim + h * vdim;
   const float og = a.gate ? sigmoidf_(a.gate[(size_t)b * a.gate_ld + h]) : 1.f;
+  if (MAPS == 2 && a.splits > 1) {  // this part's sums relative to its own maximum: [B, S, H, MAPS, vdim], then (maximum, sum) [B, S, H, MAPS, 2]
+    const size_t row = (((size_t)b * gridDim.z + blockIdx.z) * a.H + h) * MAPS;
+    float* ml = a.scratch + (size_t)gridDim.x * gridDim.z * a.H * MAPS * vdim;
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) {
+      const float *mm = ms + mp * 2 * STK_DW, *ow = os + mp * STK_DW * vdim;
+      float M = mm[0], L = 0.f;
+      for (int w = 1; w < STK_DW; w++) M = fmaxf(M, mm[w]);
+      float cw[STK_DW];
+      for (int w = 0; w < STK_DW; w++) {
+        cw[w] = mm[w] > -INFINITY ? expf(mm[w] - M) : 0.f;
+        L += mm[STK_DW + w] * cw[w];
+      }
+      for (int d = tid; d < vdim; d += 64 * STK_DW) {
+        float o = 0.f;
+        for (int w = 0; w < STK_DW; w++) o += ow[w * vdim + d] * cw[w];
+        a.scratch[(row + mp) * vdim + d] = o;
+      }
+      if (tid == 0) ml[(row + mp) * 2] = M, ml[(row + mp) * 2 + 1] = L;
+    }
+    return;
+  }
   auto joined = [&](int mp, int d) {  // the waves' partial sums of channel d, in wave order
     const float *mm = ms + mp * 2 * STK_DW, *ow = os + mp * STK_DW * vdim;
     float M = mm[0];
@@ -1075,9 +1098,54 @@ __global__ __launch_bounds__(64 * STK_DW) void stk_attn_decode_kernel(StkAttnArg
   for (int d = tid; d < vdim; d += 64 * STK_DW) El<T>::st(out + d, joined(0, d) * og);
 }
 
+// the parts of a differential decode added up in order, the two maps combined, normed and stored: a workgroup per (sequence, head)
+template <typename T>
+__global__ __launch_bounds__(128) void stk_attn_decode_join_kernel(StkAttnArgs a) {
+  __shared__ float ws[2][64], red[2];
+  const int b = blockIdx.x, h = blockIdx.y, S = a.splits, vdim = a.vdim, tid = threadIdx.x, lane = tid & 63, mp = tid >> 6;
+  const float* ml = a.scratch + (size_t)gridDim.x * S * a.H * 2 * vdim;
+  {  // wave mp: the weights of map mp's parts, lane = part
+    const bool in = lane < S;
+    const size_t at = ((((size_t)b * S + (in ? lane : 0)) * a.H + h) * 2 + mp) * 2;
+    const float m = in ? ml[at] : -INFINITY, l = in ? ml[at + 1] : 0.f;
+    const float M = wave_max(m), w = m > -INFINITY ? expf(m - M) : 0.f;
+    const float L = wave_sum(w * l);
+    ws[mp][lane] = L > 0.f ? w * (mp ? a.diff_lambda : 1.f) / L : 0.f;
+  }
+  __syncthreads();
+  float o[4], q2 = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; i++) {  // (vdim <= 512)
+    const int c = tid + i * 128;
+    o[i] = 0.f;
+    if (c >= vdim) continue;
+    float o1 = 0.f, o2 = 0.f;
+    for (int s = 0; s < S; s++) {
+      const float* p = a.scratch + (((size_t)b * S + s) * a.H + h) * 2 * vdim + c;
+      o1 = fmaf(ws[0][s], p[0], o1), o2 = fmaf(ws[1][s], p[vdim], o2);
+    }
+    o[i] = o1 - o2;
+    q2 = fmaf(o[i], o[i], q2);
+  }
+  q2 = wave_sum(q2);
+  if (lane == 0) red[mp] = q2;
+  __syncthreads();
+  const float f = a.diff_scale / sqrtf((red[0] + red[1]) / (float)vdim + a.diff_eps);
+  T* out = (T*)a.out + ((size_t)b * a.H + h) * vdim;
+#pragma unroll
+  for (int i = 0; i < 4; i++)
+    if (tid + i * 128 < vdim) El<T>::st(out + tid + i * 128, o[i] * f);
+}
+
 }  // namespace
 
 // ================================================================================================ launchers
+int vra_stack_diff_splits(int max_len, int max_seqs, int heads, int vdim) {
+  int s = max_len > 512 ? 8 : 1;
+  while (s > 1 && (int64_t)max_seqs * s * heads * 2 * (vdim + 2) * 4 > (int64_t)512 << 20) s--;
+  return s;
+}
+
 int vra_stack_gemm_granule(int rows, int groups) { return groups > 0 && rows / groups >= 128 ? 64 : 16; }
 
 void vra_stack_gemm(const StkGemmArgs& g, int dtype, int64_t stream) {
@@ -1087,7 +1155,9 @@ void vra_stack_gemm(const StkGemmArgs& g, int dtype, int64_t stream) {
   VRA_CHECK_ARG(g.batch >= 1 && (g.batch == 1 || !g.tile_group), "stack gemm: a batched product has no row groups");
   hipStream_t st = as_stream(stream);
   const int nb = g.batch;
-  const bool big = g.tile_group ? g.granule == 64 : g.M > 32;
+  // (few columns over a long K, the first stage of a low-rank projection: the 64-row tiles would leave most of the chip idle)
+  const bool narrow = dtype == VRA_BF16 && !g.tile_group && !g.a_scale && nb == 1 && g.N <= 128 && g.K >= 1024 && g.M <= 8192;
+  const bool big = g.tile_group ? g.granule == 64 : g.M > 32 && !narrow;
   const bool mfma = dtype == VRA_BF16 && g.K % 8 == 0 && g.lda % 8 == 0 && ((uintptr_t)g.a % 16 == 0) && ((uintptr_t)g.w % 16 == 0) &&
                     (g.w_group_stride % 8 == 0) && (g.a_batch_stride % 8 == 0) && (g.w_batch_stride % 8 == 0);
   VRA_CHECK_ARG(g.epi >= 0 && g.epi <= 2 && (g.epi != 2 || (g.act >= 3 && g.act <= 6)) && (g.softcap <= 0.f || g.epi != 1), "stack gemm: unknown epilogue");
@@ -1201,11 +1271,15 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
     if (!two && vra_stack_latent_decode(a, dtype, stream)) return;
     const size_t lds = (std::max<size_t>(dm, STK_DW) + (a.maps + 1) * STK_DW * 64 + a.maps * (2 * STK_DW + STK_DW * (size_t)a.vdim)) * sizeof(float);
     VRA_CHECK_ARG(lds <= 64 * 1024, "stack attention: head does not fit LDS");
-    dim3 grid(a.B, a.H);
+    StkAttnArgs k = a;
+    if (!two || !k.scratch || k.splits < 1) k.splits = 1;
+    VRA_CHECK_ARG(k.splits <= 64 && (k.splits == 1 || (size_t)a.B * k.splits * a.H * 2 * (a.vdim + 2) * sizeof(float) <= a.scratch_bytes),
+                  "stack attention: at most 64 parts, and their scratch");
+    dim3 grid(a.B, a.H, k.splits);
 #define STK_DEC(TT, NRV)                                                                              \
   launch_checked("stack attention (decode)", [&] {                                                    \
-    if (two) stk_attn_decode_kernel<TT, NRV, 2><<<grid, 64 * STK_DW, lds, st>>>(a);                   \
-    else stk_attn_decode_kernel<TT, NRV, 1><<<grid, 64 * STK_DW, lds, st>>>(a);                       \
+    if (two) stk_attn_decode_kernel<TT, NRV, 2><<<grid, 64 * STK_DW, lds, st>>>(k);                   \
+    else stk_attn_decode_kernel<TT, NRV, 1><<<grid, 64 * STK_DW, lds, st>>>(k);                       \
   })
     if (dtype == VRA_F32) {
       if (a.vdim <= 256) STK_DEC(float, 4);
@@ -1215,6 +1289,11 @@ void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream) {
       else STK_DEC(uint16_t, 8);
     }
 #undef STK_DEC
+    if (k.splits > 1)
+      launch_checked("stack attention (join)", [&] {
+        if (dtype == VRA_F32) stk_attn_decode_join_kernel<float><<<dim3(a.B, a.H), 128, 0, st>>>(k);
+        else stk_attn_decode_join_kernel<uint16_t><<<dim3(a.B, a.H), 128, 0, st>>>(k);
+      });
     return;
   }
   if (!two && vra_stack_latent_prefill(a, dtype, stream)) return;
@@ -1330,4 +1409,17 @@ extern "C" void vra_stack_op_gemm_post(const void* a, int32_t lda, const void* w
   g.alpha = alpha, g.bias = bias, g.tile_group = tile_group, g.granule = granule, g.a_row = a_row, g.out_row = out_row, g.epi = epi, g.act = act;
   g.softcap = softcap;
   vra_stack_gemm(g, dtype, stream);
+}
+// two maps per head over the same values, combined and normed (decode form: with scratch the key range in `splits` parts)
+extern "C" void vra_stack_op_attention_differential(const void* q, int32_t ldq, void* out, const void* kc, const void* vc, const int64_t* positions,
+                                                    const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_q, int32_t B, int32_t T,
+                                                    int32_t max_q, int32_t H, int32_t G, int32_t dim, int32_t vdim, int32_t BS, int32_t max_blocks,
+                                                    float scale, float lambda, float eps, float out_scale, float* scratch, int64_t scratch_bytes,
+                                                    int32_t splits, int32_t dtype, int64_t stream) {
+  StkAttnArgs a;
+  a.q = q, a.ldq = ldq, a.out = out, a.kc = kc, a.vc = vc, a.positions = positions, a.block_tables = block_tables, a.context_lens = context_lens;
+  a.cu_q = cu_q, a.B = B, a.T = T, a.max_q = max_q, a.H = H, a.G = G, a.dim = dim, a.vdim = vdim, a.BS = BS, a.max_blocks = max_blocks;
+  a.scale = scale, a.maps = 2, a.diff_lambda = lambda, a.diff_eps = eps, a.diff_scale = out_scale;
+  a.scratch = scratch, a.scratch_bytes = (size_t)scratch_bytes, a.splits = splits;
+  vra_stack_attention(a, dtype, stream);
 }

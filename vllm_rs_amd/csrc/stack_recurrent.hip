@@ -932,7 +932,7 @@ __global__ __launch_bounds__(256) void stk_head_norm_gate_kernel(const float* o,
     }
     return;
   }
-  for (int h = wave; h < H; h += 4) {
+  for (int h = blockIdx.y * 4 + wave; h < H; h += 4 * gridDim.y) {
     const float* src = o + ((size_t)t * H + h) * vdim;
     float s = 0.f;
     for (int c = lane; c < vdim; c += 64) s = fmaf(src[c], src[c], s);
@@ -1242,11 +1242,12 @@ void vra_stack_linear_scan(const StkScanArgs& a, int64_t stream) {
 void vra_stack_head_norm_gate(const float* o, const float* w, const float* gate, int gate_ld, int gate_act, float eps, void* out, int T, int H, int vdim,
                               int dtype, int64_t stream, int w_per_head) {
   VRA_CHECK_ARG(o && out && T > 0 && H > 0 && vdim > 0, "stack head norm: null pointer or empty shape");
+  const dim3 grid(T, std::min((H + 3) / 4, 64));  // a head per wave
   if (dtype == VRA_F32)
-    launch_checked("stack head norm", [&] { stk_head_norm_gate_kernel<float><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (float*)out, H, vdim, w_per_head); });
+    launch_checked("stack head norm", [&] { stk_head_norm_gate_kernel<float><<<grid, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (float*)out, H, vdim, w_per_head); });
   else
     launch_checked("stack head norm", [&] {
-      stk_head_norm_gate_kernel<uint16_t><<<T, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (uint16_t*)out, H, vdim, w_per_head);
+      stk_head_norm_gate_kernel<uint16_t><<<grid, 256, 0, as_stream(stream)>>>(o, w, gate, gate_ld, gate_act, eps, (uint16_t*)out, H, vdim, w_per_head);
     });
 }
 
@@ -1381,4 +1382,35 @@ extern "C" void vra_stack_op_linear_scan_ex(const float* q, int32_t ldq, const f
   a.head_decay = head_decay, a.beta = beta, a.ldb = ldb, a.q_scale = q_scale, a.state = state, a.state_slots = state_slots, a.positions = positions;
   a.cu_q = cu_q, a.out = out, a.ldo = ldo, a.B = B, a.H = H, a.qk_rep = qk_rep, a.dim = dim, a.vdim = vdim;
   vra_stack_linear_scan(a, stream);
+}
+// token shift, the bonus recurrence, the per-head output norm, and the seam of blocks whose sub-blocks read the residual stream itself
+extern "C" void vra_stack_op_token_shift(const float* x, const float* mu, int32_t n, float* shift_state, const int64_t* positions, const uint32_t* cu_q,
+                                         const int32_t* state_slots, void* out, int32_t T, int32_t B, int32_t W, int32_t dtype, int64_t stream) {
+  StkShiftArgs a;
+  a.x = x, a.mu = mu, a.n = n, a.shift_state = shift_state, a.positions = positions, a.cu_q = cu_q, a.state_slots = state_slots, a.out = out;
+  a.T = T, a.B = B, a.W = W;
+  vra_stack_token_shift(a, dtype, stream);
+}
+extern "C" void vra_stack_op_bonus_scan(const float* q, int32_t ldq, const float* k, int32_t ldk, const float* v, int32_t ldv, const float* decay, int32_t ldd,
+                                        const float* bonus, float q_scale, float* state, const int32_t* state_slots, const int64_t* positions,
+                                        const uint32_t* cu_q, float* out, int32_t ldo, int32_t B, int32_t H, int32_t qk_rep, int32_t dim, int32_t vdim,
+                                        int64_t stream) {
+  StkScanArgs a;
+  a.q = q, a.ldq = ldq, a.k = k, a.ldk = ldk, a.v = v, a.ldv = ldv, a.decay = decay, a.ldd = ldd, a.bonus = bonus, a.q_scale = q_scale, a.state = state;
+  a.state_slots = state_slots, a.positions = positions, a.cu_q = cu_q, a.out = out, a.ldo = ldo, a.B = B, a.H = H, a.qk_rep = qk_rep, a.dim = dim, a.vdim = vdim;
+  vra_stack_linear_scan(a, stream);
+}
+extern "C" void vra_stack_op_head_norm_gate(const float* o, const float* w, int32_t w_per_head, const float* gate, int32_t gate_ld, int32_t gate_act, float eps,
+                                            void* out, int32_t T, int32_t H, int32_t vdim, int32_t dtype, int64_t stream) {
+  vra_stack_head_norm_gate(o, w, gate, gate_ld, gate_act, eps, out, T, H, vdim, dtype, stream, w_per_head);
+}
+extern "C" void vra_stack_op_seam_post(float* x, const float* p1, int32_t n1, const float* pw, const int32_t* pe, const float* p2, const float* xw,
+                                       const float* post_w, void* h, float eps, int32_t T, int32_t W, const void* router_w, const float* router_bias,
+                                       int32_t n_router, int32_t top, int32_t n_identity, float weight_scale, int32_t* pair_expert, float* pair_weight,
+                                       float* id_weight, int32_t dtype, int64_t stream) {
+  StkSandwichArgs a;
+  a.x = x, a.p1 = p1, a.n1 = n1, a.pw = pw, a.pe = pe, a.p2 = p2, a.xw = xw, a.post_w = post_w, a.h = h, a.eps = eps, a.T = T, a.W = W, a.pre_identity = h != nullptr;
+  a.router_w = router_w, a.router_bias = router_bias, a.router_kind = 1, a.n_router = n_router, a.top = top, a.n_identity = n_identity;
+  a.weight_scale = weight_scale, a.pair_expert = pair_expert, a.pair_weight = pair_weight, a.id_weight = id_weight;
+  vra_stack_sandwich_norm(a, dtype, stream);
 }

@@ -287,7 +287,7 @@ class StackModel : public ModelBase {
   float *pair_weight_ = nullptr, *row_scale_ = nullptr, *gate_ = nullptr;
   float* sig_scratch_ = nullptr;
   size_t sig_scratch_bytes_ = 0;
-  float* lat_scratch_ = nullptr;  // decoded tokens of latent layers: partial sums over parts of the key range
+  float* lat_scratch_ = nullptr;  // decoded tokens of latent and differential layers: partial sums over parts of the key range
   size_t lat_scratch_bytes_ = 0;
   bool trace_on_ = false;
   float* trace_ = nullptr;

@@ -1,5 +1,6 @@
-"""Throughput of a layer-stack model (Ditilix, Gaperax, Zifetar, Sudosun or Pesivik design) beside the dense bf16 Llama of the same widths —
-`python bench.py --design ditilix|gaperax|zifetar|sudosun|pesivik` (Pesivik also beside a Gaperax stack whose layers are all latent attention
+"""Throughput of a layer-stack model (Ditilix, Gaperax, Zifetar, Sudosun, Pesivik or Kemavik design) beside the dense bf16 Llama of the same widths —
+`python bench.py --design ditilix|gaperax|zifetar|sudosun|pesivik|kemavik` (Kemavik also beside the Ditilix mixture of experts of the same widths,
+which is softmax attention with borrowed keys, and beside the Zifetar design, whose recurrences have decays per key channel; Pesivik also beside a Gaperax stack whose layers are all latent attention
 with the same latents, and beside the Sudosun design of the same widths and experts; Sudosun also beside the Zifetar design of the same widths, its closest model;
 Zifetar also beside the Ditilix mixture of experts of the same widths, the closest
 model of its class).
@@ -174,6 +175,38 @@ def pesivik_costs(cj):
     return 2 * n, 2 * n
 
 
+def kemavik_config(width, heads, kv_heads, dim, vdim, r_heads, r_dim, rank, layers, vocab, experts, top, expert_ff, shared_ff):
+    """config.json dict of a Kemavik model: layers in the order differential attention, the same with the first one's keys and values, time mixing;
+    every layer a mixture of experts with a shared one (four identity experts beside the real ones)"""
+    ls = []
+    for i in range(layers):
+        at = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, diff=0.4)
+        if i % 3 == 1:
+            at["kv_from"] = i - 1
+        mlp = dict(kind="moe", expert=dict(ff=expert_ff), router=dict(experts=experts, top=top, identity=4, scale=2.0), shared=dict(ff=shared_ff))
+        ls.append(dict(type="wkv", mixer=dict(heads=r_heads, dim=r_dim, rank=rank), mlp=mlp) if i % 3 == 2 else dict(type="attention", mixer=at, mlp=mlp))
+    return dict(architecture="Kemavik", width=width, vocab=vocab, norm=dict(eps=1e-6), layers=ls)
+
+
+def kemavik_costs(cj):
+    """(matrix FLOPs per token without attention and recurrences, weight bytes a one-token step reads) of a Kemavik config"""
+    W, n = cj["width"], 0
+    for layer in cj["layers"]:
+        mx, mlp = layer["mixer"], layer.get("mlp")
+        if layer["type"] == "wkv":
+            m = mx["heads"] * mx["dim"]
+            n += 5 * W * m + mx["rank"] * (W + m)
+        else:
+            H, G, D, V = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+            n += W * (2 * H * D + (0 if mx.get("kv_from") is not None else 2 * G * D + G * V)) + H * V * W
+        if mlp and mlp["kind"] == "moe":
+            n += mlp["router"]["top"] * 3 * W * mlp["expert"]["ff"] + W * (mlp["router"]["experts"] + mlp["router"]["identity"]) + 3 * W * mlp["shared"]["ff"]
+        elif mlp:
+            n += 2 * W * mlp["ff"]
+    n += cj["vocab"] * W
+    return 2 * n, 2 * n
+
+
 def latent_gaperax_config(width, heads, dim, ff, layers, vocab, kv_rank, q_rank, rot_dim):
     """a Gaperax stack whose layers are all latent attention"""
     cj = gaperax_config(width, heads, heads, dim, ff, layers, vocab, kv_rank, q_rank, rot_dim, 0, 0)
@@ -259,14 +292,26 @@ PESIVIK_SIZES = {
 }
 
 
+KEMAVIK_SIZES = {
+    # name: (width, heads, kv_heads, size of a map, value size, heads and head size of the time mixing, its rank, layers, vocab, experts, top,
+    #        expert ff, shared ff)
+    "kemavik-2048": (2048, 16, 4, 64, 128, 16, 128, 64, 3, 32000, 16, 2, 1024, 2048),
+    "kemavik-4096": (4096, 32, 8, 64, 128, 32, 128, 128, 3, 32000, 16, 2, 2048, 2048),
+}
+
+
 def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design="ditilix"):
     from . import _lib, checkpoint
     from .engine import BF16, Engine
     L = _lib.load()
     lines = []
-    table = GAPERAX_SIZES if design == "gaperax" else (ZIFETAR_SIZES if design == "zifetar" else (SUDOSUN_SIZES if design == "sudosun" else (PESIVIK_SIZES if design == "pesivik" else SIZES)))
+    table = GAPERAX_SIZES if design == "gaperax" else (ZIFETAR_SIZES if design == "zifetar" else (SUDOSUN_SIZES if design == "sudosun" else (PESIVIK_SIZES if design == "pesivik" else (KEMAVIK_SIZES if design == "kemavik" else SIZES))))
     for name in (sizes or table):
-        if design == "pesivik":
+        if design == "kemavik":
+            width, heads, kvh, dim, vdim, rh, rd, rank, layers, vocab, experts, top, eff, sff = table[name]
+            cj = kemavik_config(width, heads, kvh, dim, vdim, rh, rd, rank, layers, vocab, experts, top, eff, sff)
+            dim, ff = vdim, 4 * width
+        elif design == "pesivik":
             width, heads, dim, layers, vocab, kr, qr, rd, window, experts, top, eff, sff, groups, keep = table[name]
             cj = pesivik_config(width, heads, dim, layers, vocab, kr, qr, rd, window, experts, top, eff, sff, groups, keep)
             kvh, ff = heads // 4, 4 * width
@@ -288,7 +333,18 @@ def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design
         res = dict(stack=measure(eng, L, vocab, prefill_tokens, steps, warmup))
         eng.close()
         res["stack"]["flops_per_token"], res["stack"]["weight_bytes_per_step"] = (
-            pesivik_costs(cj) if design == "pesivik" else (sudosun_costs(cj) if design == "sudosun" else (zifetar_costs(cj) if design == "zifetar" else (gaperax_costs(cj) if design == "gaperax" else stack_costs(cj)))))
+            kemavik_costs(cj) if design == "kemavik" else pesivik_costs(cj) if design == "pesivik" else (sudosun_costs(cj) if design == "sudosun" else (zifetar_costs(cj) if design == "zifetar" else (gaperax_costs(cj) if design == "gaperax" else stack_costs(cj)))))
+        if design == "kemavik":  # the closest models: softmax attention with borrowed keys and the same experts; recurrences with per-channel decays
+            dj = stack_config(width, heads, kvh, dim, ff, layers + 1, vocab, experts, top, eff, sff, False)
+            dj["layers"] = dj["layers"][1:]
+            for i in range(1, layers, 3):
+                dj["layers"][i] = dict(dj["layers"][i], mixer=dict(dj["layers"][i]["mixer"], kv_from=i - 1))
+            zj = zifetar_config(width, heads, kvh, dim, layers, vocab, experts, top, eff, 4096, rank)
+            for key, other, costs in (("ditilix_moe", dj, stack_costs), ("zifetar", zj, zifetar_costs)):
+                eng = Engine(checkpoint.parse_config(other), num_gpu_blocks=512, max_num_seqs=8, max_model_len=4096, use_graph=graph).init_synthetic()
+                res[key] = measure(eng, L, vocab, prefill_tokens, steps, warmup)
+                eng.close()
+                res[key]["flops_per_token"], res[key]["weight_bytes_per_step"] = costs(other)
         if design == "pesivik":  # the two closest models: latent attention with the same latents (dense gated feed-forward); the sandwich seams
             # and mixture of experts of the Sudosun design (recurrent mixers)
             gj = latent_gaperax_config(width, heads, dim, ff, layers, vocab, kr, qr, rd)
@@ -320,7 +376,7 @@ def main(steps=64, warmup=8, prefill_tokens=2048, graph=True, sizes=None, design
         for m in res.values():
             m["prefill_matrix_tflops"] = m["prefill_tokens_per_s"] * m["flops_per_token"] / 1e12
             m["decode_bs1_weight_gb_per_s"] = m["weight_bytes_per_step"] / (m["decode_bs1_ms_per_step"] / 1e3) / 1e9
-        line = dict(metric="stack_vs_dense_llama", size=name, design={"gaperax": "Gaperax", "zifetar": "Zifetar", "sudosun": "Sudosun", "pesivik": "Pesivik"}.get(design, "Ditilix"), dtype="bf16", data="synthetic", prefill_tokens=prefill_tokens,
+        line = dict(metric="stack_vs_dense_llama", size=name, design={"gaperax": "Gaperax", "zifetar": "Zifetar", "sudosun": "Sudosun", "pesivik": "Pesivik", "kemavik": "Kemavik"}.get(design, "Ditilix"), dtype="bf16", data="synthetic", prefill_tokens=prefill_tokens,
                     decode_context=512, steps=steps, **res)
         print(json.dumps(line), flush=True)
         lines.append(line)
