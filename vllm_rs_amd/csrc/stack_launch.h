@@ -126,8 +126,10 @@ struct StkAttnArgs {
   int splits = 0;
 };
 void vra_stack_attention(const StkAttnArgs& a, int dtype, int64_t stream);
-// parts of the key range the differential decode form takes (a model's constants: it fixes the order of the sums)
-int vra_stack_diff_splits(int max_len, int max_seqs, int heads, int vdim);
+// parts of the key range the differential decode form takes for a batch of B sequences (few heads a step: more parts, so that a long context spreads
+// over the chip), and the scratch that holds them for any batch up to max_seqs
+int vra_stack_diff_splits(int max_len, int B, int heads);
+size_t vra_stack_diff_scratch(int max_len, int max_seqs, int heads, int vdim);
 // its shared-row form on the matrix cores (stack_latent.hip): bf16 prompt steps with G = 1 and vc = kc, rows up to 576 wide, values up to 512;
 // false: not a shape of that kernel, nothing was launched
 // vra_stack_latent_decode: the same for one token per sequence, in two launches over `splits` parts of the key range (any number from 1 to 64; it

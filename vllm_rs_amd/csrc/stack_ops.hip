@@ -667,7 +667,7 @@ __global__ __launch_bounds__(256) void stk_attn_prefill_kernel(StkAttnArgs a) {
 // kernel), all eight share the transposed V tile; at the end the second map's rows travel through LDS to the first map's waves, which
 // combine, norm and store.
 template <int DC, int VT, int MAPS>
-__global__ __launch_bounds__(256 * MAPS) void stk_attn_prefill_mfma_kernel(StkAttnArgs a) {
+__global__ __launch_bounds__(256 * MAPS, MAPS == 2 && DC <= 2 ? 4 : 1) void stk_attn_prefill_mfma_kernel(StkAttnArgs a) {
   constexpr int KT = 32, VLD = KT + 8;  // LDS row of a value channel: 32 positions + 8 (rows stay 16-byte aligned, lanes spread over banks)
   constexpr int NT = 256 * MAPS, XT = VT < 4 ? VT : 4;  // threads; channel tiles handed over at a time (MAPS 2: 4 waves x 64 lanes x 16 bytes each)
   constexpr int VT_BYTES = VT * 16 * VLD * 2, X_BYTES = MAPS == 2 ? XT * 4096 : 0;
@@ -834,15 +834,19 @@ __global__ __launch_bounds__(256 * MAPS) void stk_attn_prefill_mfma_kernel(StkAt
     for (int t = 0; t < VT; t++) {
       acc[t][0] *= corr, acc[t][1] *= corr, acc[t][2] *= corr, acc[t][3] *= corr;
     }
-    u32x4 vf[VT];
+    // heads of four channel tiles first, then their tails: the two MFMAs into one accumulator are four instructions apart, and only four V
+    // fragments are held at a time (fully unrolled: every accumulator keeps its registers, no indexed register moves next to an MFMA)
+    constexpr int VG = 4;
 #pragma unroll
-    for (int t = 0; t < VT; t++) vf[t] = *(const u32x4*)(vt + (t * 16 + rq) * VLD + oct * 8);
-    // heads of all channel tiles first, then the tails: the two MFMAs into one accumulator are VT instructions apart
-    // (fully unrolled: every accumulator keeps its registers, no indexed register moves next to an MFMA)
+    for (int t0_ = 0; t0_ < VT; t0_ += VG) {
+      u32x4 vf[VG];
 #pragma unroll
-    for (int t = 0; t < VT; t++) BF16::mfma(acc[t], __builtin_bit_cast(s16x8, vf[t]), __builtin_bit_cast(s16x8, phi));
+      for (int t = 0; t < VG; t++) vf[t] = *(const u32x4*)(vt + ((t0_ + t) * 16 + rq) * VLD + oct * 8);
 #pragma unroll
-    for (int t = 0; t < VT; t++) BF16::mfma(acc[t], __builtin_bit_cast(s16x8, vf[t]), __builtin_bit_cast(s16x8, plo));
+      for (int t = 0; t < VG; t++) BF16::mfma(acc[t0_ + t], __builtin_bit_cast(s16x8, vf[t]), __builtin_bit_cast(s16x8, phi));
+#pragma unroll
+      for (int t = 0; t < VG; t++) BF16::mfma(acc[t0_ + t], __builtin_bit_cast(s16x8, vf[t]), __builtin_bit_cast(s16x8, plo));
+    }
     VRA_MFMA_DRAIN();
   }
   l += __shfl_xor(l, 16, 64);
@@ -1140,10 +1144,10 @@ __global__ __launch_bounds__(128) void stk_attn_decode_join_kernel(StkAttnArgs a
 }  // namespace
 
 // ================================================================================================ launchers
-int vra_stack_diff_splits(int max_len, int max_seqs, int heads, int vdim) {
-  int s = max_len > 512 ? 8 : 1;
-  while (s > 1 && (int64_t)max_seqs * s * heads * 2 * (vdim + 2) * 4 > (int64_t)512 << 20) s--;
-  return s;
+#define STK_DIFF_PARTS 512  // (sequence, head, part) workgroups a decode step aims at
+int vra_stack_diff_splits(int max_len, int B, int heads) { return max_len > 512 ? std::min(8, std::max(1, STK_DIFF_PARTS / std::max(B * heads, 1))) : 1; }
+size_t vra_stack_diff_scratch(int max_len, int max_seqs, int heads, int vdim) {  // (more than one part: B * heads * parts <= STK_DIFF_PARTS)
+  return vra_stack_diff_splits(max_len, 1, heads) > 1 ? (size_t)STK_DIFF_PARTS * 2 * (vdim + 2) * sizeof(float) : 0;
 }
 
 int vra_stack_gemm_granule(int rows, int groups) { return groups > 0 && rows / groups >= 128 ? 64 : 16; }

@@ -1044,9 +1044,7 @@ bool StackModel::init_buffers(int max_tokens, int max_seqs) {
     lat_scratch_bytes_ = std::max(lat_scratch_bytes_, (size_t)max_seqs * s * L.heads * (L.kv_rank + 2) * 4);
   }
   for (const StackLayer& L : layers_) {
-    if (L.mixer != 7) continue;
-    const int s = vra_stack_diff_splits(mc_.max_position_embeddings, max_seqs, L.heads, L.vdim);
-    if (s > 1) lat_scratch_bytes_ = std::max(lat_scratch_bytes_, (size_t)max_seqs * s * L.heads * 2 * (L.vdim + 2) * 4);
+    if (L.mixer == 7) lat_scratch_bytes_ = std::max(lat_scratch_bytes_, vra_stack_diff_scratch(mc_.max_position_embeddings, max_seqs, L.heads, L.vdim));
   }
   if (lat_scratch_bytes_ && !(lat_scratch_ = (float*)dalloc(lat_scratch_bytes_))) return false;
   if (nmix && !(mix_ = dalloc(nmix * T * W * es_))) return false;
@@ -1587,7 +1585,7 @@ bool StackModel::mixer_differential(const StackLayer& L, const InputMetadata& md
   a.cu_q = md.is_prefill ? md.cu_seqlens_q : nullptr;
   a.B = md.n_seqs, a.T = T, a.max_q = md.is_prefill ? md.max_seqlen_q : 1, a.H = H, a.G = L.kv_heads, a.dim = L.dim, a.vdim = L.vdim;
   a.BS = ec_.block_size, a.max_blocks = md.max_blocks, a.scale = L.scale;
-  a.scratch = lat_scratch_, a.scratch_bytes = lat_scratch_bytes_, a.splits = vra_stack_diff_splits(mc_.max_position_embeddings, max_seqs_, H, L.vdim);
+  a.scratch = lat_scratch_, a.scratch_bytes = lat_scratch_bytes_, a.splits = vra_stack_diff_splits(mc_.max_position_embeddings, md.n_seqs, H);
   a.maps = 2, a.diff_lambda = L.lambda, a.diff_eps = eps_, a.diff_scale = 1.f - L.diff;
   vra_stack_attention(a, dt_, stream);
   StkGemmArgs o;
